@@ -30,7 +30,7 @@ class ChunkMask:
 
 @dataclasses.dataclass(frozen=True)
 class WaveScaling:
-    """Slowing the rotation's long waves down (see ``parts.attention.rotation_frequencies``)."""
+    """Slowing the rotation's long waves down (see ``parts.position.rotation_frequencies``)."""
     factor: float = key(convert=as_float)
     original: float = key(convert=as_float)
     fast: float = key(convert=as_float)

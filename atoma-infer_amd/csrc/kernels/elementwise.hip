@@ -3,6 +3,7 @@
 // types only decide how values are read and stored.
 #include "common.h"
 #include "cache_layout.h"
+#include "gate_act.h"
 
 using namespace atoma;
 
@@ -34,7 +35,7 @@ __device__ __forceinline__ void store4(bf16_t* p, const f4& a) {
 // Reference: models/src/llama.rs:470 (candle Embedding).
 template <typename TW>
 __global__ void embed_kernel(const int32_t* __restrict__ tokens, const TW* __restrict__ table,
-                             float* __restrict__ out, int width, int vocab) {
+                             float* __restrict__ out, int width, int vocab, float scale) {
   const int t = blockIdx.x;
   const int token = tokens[t];
   const size_t dst = (size_t)t * width;
@@ -43,18 +44,19 @@ __global__ void embed_kernel(const int32_t* __restrict__ tokens, const TW* __res
     return;
   }
   const size_t src = (size_t)token * width;
-  for (int i = threadIdx.x; i < width; i += blockDim.x) out[dst + i] = to_f32(table[src + i]);
+  for (int i = threadIdx.x; i < width; i += blockDim.x) out[dst + i] = to_f32(table[src + i]) * scale;
 }
 
 extern "C" int atoma_embed(const int32_t* tokens, const void* table, int table_dtype, float* out, int n_tokens,
-                           int width, int vocab, hipStream_t stream) {
+                           int width, int vocab, float scale, hipStream_t stream) {
   if (n_tokens <= 0) return 0;
   dim3 grid(n_tokens), block(256);
   if (table_dtype == kF32)
-    hipLaunchKernelGGL(embed_kernel<float>, grid, block, 0, stream, tokens, (const float*)table, out, width, vocab);
+    hipLaunchKernelGGL(embed_kernel<float>, grid, block, 0, stream, tokens, (const float*)table, out, width, vocab,
+                       scale);
   else if (table_dtype == kBF16)
     hipLaunchKernelGGL(embed_kernel<bf16_t>, grid, block, 0, stream, tokens, (const bf16_t*)table, out, width,
-                       vocab);
+                       vocab, scale);
   else
     return ATOMA_ERR_DTYPE;
   ATOMA_LAUNCH_CHECK();
@@ -66,14 +68,14 @@ extern "C" int atoma_embed(const int32_t* tokens, const void* table, int table_d
 // at most 16 rows; the products are in gemm_bf16.hip).  "Begun" is: u = residual * norm weight, as bfloat16, and the
 // row's sum of squares in shares ss [parts][16]; "finished" is the division by sqrt(sum / width + eps).
 
-// Embedding gather with the first norm begun: resid [T][width] float32, u [T][width] bfloat16, ss [1][16].
+// Embedding gather (rows times `scale`) with the first norm begun: resid [T][width] float32, u [T][width] bfloat16, ss [1][16].
 // One block of 256 threads per row, 16 blocks: those beyond T only clear their share.  Four columns a thread at a
 // time where the row allows 8- and 16-byte accesses (VEC), one otherwise.
 template <typename TW, typename TG, bool VEC>
 __global__ void __launch_bounds__(256)
 embed_begin_norm_kernel(const int32_t* __restrict__ tokens, const TW* __restrict__ table, float* __restrict__ resid,
                         const TG* __restrict__ gamma, bf16_t* __restrict__ u, float* __restrict__ ss, int n_tokens,
-                        int width, int vocab) {
+                        int width, int vocab, float scale) {
   __shared__ float scratch[4];
   const int t = blockIdx.x;
   if (t >= n_tokens) {
@@ -92,7 +94,7 @@ embed_begin_norm_kernel(const int32_t* __restrict__ tokens, const TW* __restrict
       f4 o;
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
-        if (!ok) v.v[j] = nan;
+        v.v[j] = ok ? v.v[j] * scale : nan;
         o.v[j] = v.v[j] * g.v[j];
         sq += v.v[j] * v.v[j];
       }
@@ -101,7 +103,7 @@ embed_begin_norm_kernel(const int32_t* __restrict__ tokens, const TW* __restrict
     }
   } else {
     for (int i = threadIdx.x; i < width; i += 256) {
-      const float v = ok ? to_f32(table[src + i]) : nan;
+      const float v = ok ? to_f32(table[src + i]) * scale : nan;
       resid[dst + i] = v;
       u[dst + i] = from_f32<bf16_t>(v * to_f32(gamma[i]));
       sq += v * v;
@@ -113,7 +115,7 @@ embed_begin_norm_kernel(const int32_t* __restrict__ tokens, const TW* __restrict
 
 extern "C" int atoma_embed_begin_norm(const int32_t* tokens, const void* table, int table_dtype, float* resid,
                                       const void* gamma, int gamma_dtype, void* u, float* ss, int n_tokens, int width,
-                                      int vocab, hipStream_t stream) {
+                                      int vocab, float scale, hipStream_t stream) {
   if (n_tokens <= 0) return 0;
   if (n_tokens > 16) return ATOMA_ERR_SHAPE;
   const bool vec = width % 4 == 0 && (((uintptr_t)table | (uintptr_t)gamma | (uintptr_t)resid | (uintptr_t)u) & 15) == 0;
@@ -121,10 +123,12 @@ extern "C" int atoma_embed_begin_norm(const int32_t* tokens, const void* table, 
   do {                                                                                                              \
     if (vec)                                                                                                        \
       hipLaunchKernelGGL((embed_begin_norm_kernel<TW, TG, true>), dim3(16), dim3(256), 0, stream, tokens,           \
-                         (const TW*)table, resid, (const TG*)gamma, (bf16_t*)u, ss, n_tokens, width, vocab);        \
+                         (const TW*)table, resid, (const TG*)gamma, (bf16_t*)u, ss, n_tokens, width, vocab,  \
+                         scale);        \
     else                                                                                                            \
       hipLaunchKernelGGL((embed_begin_norm_kernel<TW, TG, false>), dim3(16), dim3(256), 0, stream, tokens,          \
-                         (const TW*)table, resid, (const TG*)gamma, (bf16_t*)u, ss, n_tokens, width, vocab);        \
+                         (const TW*)table, resid, (const TG*)gamma, (bf16_t*)u, ss, n_tokens, width, vocab,  \
+                         scale);        \
   } while (0)
   if (table_dtype == kF32 && gamma_dtype == kF32) ATOMA_EBN(float, float);
   else if (table_dtype == kF32 && gamma_dtype == kBF16) ATOMA_EBN(float, bf16_t);
@@ -542,7 +546,7 @@ extern "C" int atoma_rope_cache_write(void* qkv, int act_dtype, int row_stride, 
 }
 
 // ---------------------------------------------------------------------------------------------
-// out[t, i] = silu(gate[t, i]) * up[t, i], silu(z) = z * sigmoid(z); gate and up come in one row of 2 * inter.
+// out[t, i] = act(gate[t, i], up[t, i]), silu(gate) * up and its relatives (gate_act.h); gate and up come in one row of 2 * inter.
 // Reference: models/src/llama.rs:364.
 // Where gate and up of output i lie in a row of 2 * inter values: in two halves (block == 0), or interleaved in
 // blocks of 16 gate values followed by their 16 up values (block == 16), the layout of the fused gate-up product.
@@ -551,27 +555,22 @@ __device__ __forceinline__ int up_index(int i, int inter, int block) {
   return block ? ((i >> 4) << 5) + 16 + (i & 15) : inter + i;
 }
 
-// the gate's activation: 0 silu, 1 the tanh form of gelu, 0.5 g (1 + tanh(sqrt(2 / pi) (g + 0.044715 g^3)))
-__device__ __forceinline__ float gate_act(float g, int act) {
-  if (act == 1) return 0.5f * g * (1.0f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g)));
-  return g / (1.0f + expf(-g));
-}
-
 template <typename T>
-__global__ void swiglu_kernel(const T* __restrict__ gu, T* __restrict__ out, int inter, size_t total, int block, int act) {
+__global__ void swiglu_kernel(const T* __restrict__ gu, T* __restrict__ out, int inter, size_t total, int block,
+                              GateAct act) {
   for (size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x; idx < total; idx += (size_t)gridDim.x * blockDim.x) {
     const size_t t = idx / inter;
     const int i = (int)(idx % inter);
     const float g = to_f32(gu[t * 2 * inter + gate_index(i, block)]);
     const float u = to_f32(gu[t * 2 * inter + up_index(i, inter, block)]);
-    out[idx] = from_f32<T>(gate_act(g, act) * u);
+    out[idx] = from_f32<T>(gated(g, u, act));
   }
 }
 
 // four values per thread; needs inter % 4 == 0 and 16-byte aligned rows
 template <typename T>
 __global__ void __launch_bounds__(256)
-swiglu_vec_kernel(const T* __restrict__ gu, T* __restrict__ out, int inter, int n_tokens, int block, int act) {
+swiglu_vec_kernel(const T* __restrict__ gu, T* __restrict__ out, int inter, int n_tokens, int block, GateAct act) {
   const int quads = inter >> 2;
   const size_t total = (size_t)n_tokens * quads;
   for (size_t idx = (size_t)blockIdx.x * 256 + threadIdx.x; idx < total; idx += (size_t)gridDim.x * 256) {
@@ -581,14 +580,15 @@ swiglu_vec_kernel(const T* __restrict__ gu, T* __restrict__ out, int inter, int 
     const f4 u = load4(gu + t * 2 * inter + up_index(i, inter, block));
     f4 o;
 #pragma unroll
-    for (int e = 0; e < 4; ++e) o.v[e] = gate_act(g.v[e], act) * u.v[e];
+    for (int e = 0; e < 4; ++e) o.v[e] = gated(g.v[e], u.v[e], act);
     store4(out + t * inter + i, o);
   }
 }
 
 // eight bfloat16 values per thread (16-byte loads and stores); needs inter % 8 == 0 and 16-byte aligned rows
 __global__ void __launch_bounds__(256)
-swiglu_vec8_kernel(const uint16_t* __restrict__ gu, uint16_t* __restrict__ out, int inter, int n_tokens, int block, int act) {
+swiglu_vec8_kernel(const uint16_t* __restrict__ gu, uint16_t* __restrict__ out, int inter, int n_tokens, int block,
+                   GateAct act) {
   const int octs = inter >> 3;
   const size_t total = (size_t)n_tokens * octs;
   for (size_t idx = (size_t)blockIdx.x * 256 + threadIdx.x; idx < total; idx += (size_t)gridDim.x * 256) {
@@ -601,18 +601,16 @@ swiglu_vec8_kernel(const uint16_t* __restrict__ gu, uint16_t* __restrict__ out, 
     uint4 oraw;
     uint16_t* o = reinterpret_cast<uint16_t*>(&oraw);
 #pragma unroll
-    for (int e = 0; e < 8; ++e) {
-      const float gv = bf16_bits_to_f32(g[e]);
-      o[e] = f32_to_bf16_bits(gate_act(gv, act) * bf16_bits_to_f32(u[e]));
-    }
+    for (int e = 0; e < 8; ++e) o[e] = f32_to_bf16_bits(gated(bf16_bits_to_f32(g[e]), bf16_bits_to_f32(u[e]), act));
     *reinterpret_cast<uint4*>(out + t * inter + i) = oraw;
   }
 }
 
-extern "C" int atoma_swiglu(const void* gu, void* out, int dtype, int n_tokens, int inter, int block, int act,
-                            hipStream_t stream) {
+extern "C" int atoma_swiglu(const void* gu, void* out, int dtype, int n_tokens, int inter, int block, int kind,
+                            float limit, float slope, hipStream_t stream) {
   if (n_tokens <= 0) return 0;
-  if ((block != 0 && (block != 16 || inter % 16)) || act < 0 || act > 1) return ATOMA_ERR_SHAPE;
+  if ((block != 0 && (block != 16 || inter % 16)) || !gate_act_ok(kind, limit)) return ATOMA_ERR_SHAPE;
+  const GateAct act{kind, limit, slope};
   const size_t total = (size_t)n_tokens * inter;
   if (dtype == kBF16 && inter % 8 == 0 && ((uintptr_t)gu & 15) == 0 && ((uintptr_t)out & 15) == 0) {
     size_t octs = total / 8;

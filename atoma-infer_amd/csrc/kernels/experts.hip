@@ -2,8 +2,10 @@
 //
 //   route_topk    per token: scores = sigmoid(router logits), or their softmax over all experts, in float32; the `top`
 //                 experts with the largest score + correction[expert] (no correction: the score alone; the lower
-//                 index wins a tie) with their weights, score * scale (the correction chooses, it does not weigh):
-//                 a (token, choice) pair is a "slot", numbered token * top + choice;
+//                 index wins a tie) with their weights, score * scale (the correction chooses, it does not weigh),
+//                 or the experts with the largest logits, weighed by the softmax over the chosen logits alone (times
+//                 scale); logits may have a bias per expert.
+//                 A (token, choice) pair is a "slot", numbered token * top + choice;
 //   route_group   one workgroup: slots ordered by expert (perm), where each expert's slots start (offsets), and the
 //                 list of row tiles (expert, first place in perm) that the products below walk.  Which place a slot
 //                 gets inside its expert's range is not fixed; no result depends on it, since every row of a product
@@ -16,6 +18,7 @@
 //                 act = 2 squares what is positive of a result and drops the rest (experts without a gate: relu^2);
 //                 out_scale[slot] multiplies a result (experts whose weight applies to their output).
 #include "common.h"
+#include "gate_act.h"
 
 using namespace atoma;
 
@@ -23,23 +26,25 @@ constexpr int kTileM = 64, kTileN = 64, kStepK = 16;
 
 __global__ void __launch_bounds__(256)
 route_topk_kernel(const float* __restrict__ logits, int ld, int experts, int top, int32_t* __restrict__ ids,
-                  float* __restrict__ weights, int n_tokens, int softmax, const float* __restrict__ correction,
-                  float scale) {
+                  float* __restrict__ weights, int n_tokens, int score, const float* __restrict__ correction,
+                  float scale, const float* __restrict__ bias) {
   // a wave a token; lane l holds experts l, l + 64, ...
   const int lane = threadIdx.x & 63;
   const int t = blockIdx.x * 4 + (threadIdx.x >> 6);
   if (t >= n_tokens) return;
   constexpr int PER = 16;      // experts <= 1024
   // sc: what chooses (score, plus the correction where there is one); wt: what weighs (the score alone)
+  // score 0: sigmoid; 1: softmax over all experts; 2: the logits choose, softmax over the chosen ones (below)
   float sc[PER], wt[PER];
-  if (softmax) {
+#pragma unroll
+  for (int j = 0; j < PER; ++j) {
+    const int e = lane + j * 64;
+    wt[j] = e < experts ? logits[(size_t)t * ld + e] + (bias != nullptr ? bias[e] : 0.f) : -INFINITY;
+  }
+  if (score == 1) {
     float mx = -INFINITY;
 #pragma unroll
-    for (int j = 0; j < PER; ++j) {
-      const int e = lane + j * 64;
-      wt[j] = e < experts ? logits[(size_t)t * ld + e] : -INFINITY;
-      mx = fmaxf(mx, wt[j]);
-    }
+    for (int j = 0; j < PER; ++j) mx = fmaxf(mx, wt[j]);
     mx = wave_max(mx);
     float sum = 0.f;
 #pragma unroll
@@ -50,13 +55,11 @@ route_topk_kernel(const float* __restrict__ logits, int ld, int experts, int top
     sum = wave_sum(sum);
 #pragma unroll
     for (int j = 0; j < PER; ++j) wt[j] /= sum;
-  } else {
+  } else if (score == 0) {
 #pragma unroll
-    for (int j = 0; j < PER; ++j) {
-      const int e = lane + j * 64;
-      wt[j] = e < experts ? 1.0f / (1.0f + expf(-logits[(size_t)t * ld + e])) : 0.f;
-    }
+    for (int j = 0; j < PER; ++j) wt[j] = lane + j * 64 < experts ? 1.0f / (1.0f + expf(-wt[j])) : 0.f;
   }
+  float first = 0.f, total = 0.f, mine = 0.f;      // score 2: the largest logit, the sum, and lane c's choice c
 #pragma unroll
   for (int j = 0; j < PER; ++j) {
     const int e = lane + j * 64;
@@ -76,13 +79,24 @@ route_topk_kernel(const float* __restrict__ logits, int ld, int experts, int top
       if (ob > best || (ob == best && oa < arg)) best = ob, bw = ow, arg = oa;
     }
     if (arg >= experts) arg = c, bw = 0.f;     // logits that are no numbers: still an expert of the layer
-    if (lane == 0) {
-      ids[(size_t)t * top + c] = arg;
+    if (score == 2) {
+      if (c == 0) first = bw;
+      bw = expf(bw - first);
+      total += bw;
+      // weights of a choice wait for the sum: 64 choices a round in the wave's lanes, more through memory
+      if (top <= 64) { if (lane == c) mine = bw; }
+      else if (lane == 0) weights[(size_t)t * top + c] = bw;
+    } else if (lane == 0) {
       weights[(size_t)t * top + c] = bw * scale;
     }
+    if (lane == 0) ids[(size_t)t * top + c] = arg;
 #pragma unroll
     for (int j = 0; j < PER; ++j)
       if (lane + j * 64 == arg) sc[j] = -INFINITY;
+  }
+  if (score == 2) {
+    if (top <= 64) { if (lane < top) weights[(size_t)t * top + lane] = mine / total * scale; }
+    else if (lane == 0) { for (int c = 0; c < top; ++c) weights[(size_t)t * top + c] *= scale / total; }
   }
 }
 
@@ -208,14 +222,14 @@ gather_scale_kernel(const uint16_t* __restrict__ x, int ldx, const float* __rest
 // NS: blocks of 16 rows of the weight a wave takes.  KSUB: pieces of 32 columns of K a step (2, or 4 for tiles of 64
 // places: a decode step's tile holds a place or two, the product streams the weight, and what it needs is many bytes
 // in flight a step).
-// ACT: 0 the float32 result (times out_scale[slot] where given) by place or by slot; 1 silu(gate) * up over interleaved
-// rows, bfloat16 [places, N / 2]; 2 relu^2 of the result, bfloat16 [places, N].
+// ACT: 0 the float32 result (times out_scale[slot] where given) by place or by slot; 1 silu(gate) * up, or a relative
+// of it (gate_act.h), over interleaved rows, bfloat16 [places, N / 2]; 2 relu^2 of the result, bfloat16 [places, N].
 template <int ACT, int TM, int NS, int KSUB>
 __global__ void __launch_bounds__(256)
 expert_gemm_mfma_kernel(const uint16_t* __restrict__ a, const uint16_t* __restrict__ w, void* __restrict__ c, int ldc,
                         int N, int K, const int32_t* __restrict__ perm, const int32_t* __restrict__ offsets,
                         const int32_t* __restrict__ tiles, int top, int plane_rows,
-                        const float* __restrict__ out_scale) {
+                        const float* __restrict__ out_scale, GateAct gate) {
   constexpr bool SWIGLU = ACT == 1;
   constexpr int MS = TM / 16;          // blocks of 16 places a tile
   constexpr int KSTEP = 32 * KSUB;     // columns of K a step
@@ -306,10 +320,8 @@ expert_gemm_mfma_kernel(const uint16_t* __restrict__ a, const uint16_t* __restri
         uint16_t* dst = (uint16_t*)c + (size_t)place * ldc + n0;
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-          if (n_base + s * 16 + 16 + kg * 4 + i < N) {
-            const float g = acc[s][m][i];
-            dst[i] = f32_to_bf16_bits(g / (1.0f + expf(-g)) * acc[s + 1][m][i]);
-          }
+          if (n_base + s * 16 + 16 + kg * 4 + i < N)
+            dst[i] = f32_to_bf16_bits(gated(acc[s][m][i], acc[s + 1][m][i], gate));
         }
       }
     } else if constexpr (ACT == 2) {
@@ -388,16 +400,17 @@ extern "C" int atoma_gather_scale(const void* x, int ldx, const float* score, co
 extern "C" int atoma_expert_gemm_mfma(const void* a, const void* w, void* c, int ldc, int N, int K, const int32_t* perm,
                                       const int32_t* offsets, const int32_t* tiles, int max_tiles, int top,
                                       int plane_rows, int act, int tile_m, const float* out_scale,
-                                      hipStream_t stream) {
+                                      int gate_kind, float limit, float slope, hipStream_t stream) {
   if (max_tiles <= 0 || N <= 0) return 0;
   if (K <= 0 || K % 32 || N % 32 || (tile_m != 64 && tile_m != 128) || top <= 0 || max_tiles > 65535 || ((uintptr_t)a & 15) || ((uintptr_t)w & 15) ||
-      act < 0 || act > 2 || ldc < (act == 1 ? N / 2 : N) || (act != 0 && (plane_rows > 0 || out_scale != nullptr)))
+      act < 0 || act > 2 || !gate_act_ok(gate_kind, limit) || ldc < (act == 1 ? N / 2 : N) || (act != 0 && (plane_rows > 0 || out_scale != nullptr)))
     return ATOMA_ERR_SHAPE;
+  const GateAct gate{gate_kind, limit, slope};
   const int ns = 2;      // (four blocks a wave measured slower for tiles of 128 places: 467 against 336 us)
   dim3 grid((N + 64 * ns - 1) / (64 * ns), max_tiles), block(256);
 #define ATOMA_EGM(SW, TM_, NS_, KSUB_)                                                                           \
   hipLaunchKernelGGL((expert_gemm_mfma_kernel<SW, TM_, NS_, KSUB_>), grid, block, 0, stream, (const uint16_t*)a, \
-                     (const uint16_t*)w, c, ldc, N, K, perm, offsets, tiles, top, plane_rows, out_scale)
+                     (const uint16_t*)w, c, ldc, N, K, perm, offsets, tiles, top, plane_rows, out_scale, gate)
   if (act == 1 && tile_m == 64) ATOMA_EGM(1, 64, 2, 4);
   else if (act == 1) ATOMA_EGM(1, 128, 2, 2);
   else if (act == 2 && tile_m == 64) ATOMA_EGM(2, 64, 2, 4);
@@ -410,11 +423,14 @@ extern "C" int atoma_expert_gemm_mfma(const void* a, const void* w, void* c, int
 }
 
 extern "C" int atoma_route_topk(const float* logits, int ld, int experts, int top, int32_t* ids, float* weights,
-                                int n_tokens, int softmax, const float* correction, float scale, hipStream_t stream) {
+                                int n_tokens, int score, const float* correction, float scale, const float* bias,
+                                hipStream_t stream) {
   if (n_tokens <= 0) return 0;
-  if (experts <= 0 || experts > 1024 || top <= 0 || top > experts || ld < experts) return ATOMA_ERR_SHAPE;
+  if (experts <= 0 || experts > 1024 || top <= 0 || top > experts || ld < experts || score < 0 ||
+      score > 2)
+    return ATOMA_ERR_SHAPE;
   hipLaunchKernelGGL(route_topk_kernel, dim3((n_tokens + 3) / 4), dim3(256), 0, stream, logits, ld, experts, top, ids,
-                     weights, n_tokens, softmax, correction, scale);
+                     weights, n_tokens, score, correction, scale, bias);
   ATOMA_LAUNCH_CHECK();
   return 0;
 }

@@ -11,7 +11,7 @@
 //   latent_rope_prepare  attention over one latent vector per token with a rotated key part shared by all heads:
 //                        from [dq | dkv | g], cq = rmsnorm(dq) wq in the activation dtype; c = rmsnorm(dkv[:rank]) wc
 //                        and the rotated last `rd` columns of dkv form the cached key [c | k_rot | 0], the cached
-//                        value is [c | 0]; sigmoid(g) in float32.
+//                        value is [c | 0]; sigmoid(g) in float32 (n_gate may be 0: no gates).
 //   latent_q_rope        the queries behind their second projection: the last `rd` columns of every head rotated,
 //                        all columns to the activation dtype.
 //   gate_mul             y[t, h, j] = att[t, h, j] * gate[t, h, j] for the first vd of a head's hd_out columns.
@@ -90,7 +90,8 @@ __global__ void __launch_bounds__(256)
 latent_rope_prepare_kernel(const float* __restrict__ proj, int ld, int off_dq, int off_c, int off_g, int q_rank,
                            int rank, int rd, int rank_p, int n_gate, const float* __restrict__ wq,
                            const float* __restrict__ wc, float eps, const int32_t* __restrict__ positions,
-                           const float* __restrict__ freq, int rot, TA* __restrict__ cq, TC* __restrict__ kcache,
+                           const float* __restrict__ freq, int rot, int interleaved, TA* __restrict__ cq,
+                           TC* __restrict__ kcache,
                            TC* __restrict__ vcache, const int32_t* __restrict__ slot_mapping, int page_size,
                            float* __restrict__ gate) {
   __shared__ float scratch[4];
@@ -120,18 +121,19 @@ latent_rope_prepare_kernel(const float* __restrict__ proj, int ld, int off_dq, i
       kv = vv = p[off_c + i] * ic * wc[i];
     } else if (i < rank + rd) {
       const int d = i - rank;
-      kv = d < rot ? turned(kr, d, rot, 1, cs, sn) : kr[d];
+      kv = d < rot ? turned(kr, d, rot, interleaved, cs, sn) : kr[d];
     }
     kt[key_offset(off, i, page_size)] = from_f32<TC>(kv);
     vt[value_offset(i, off, rank_p, page_size)] = from_f32<TC>(vv);
   }
 }
 
-// q float32 [T, heads (dim + rd)] -> the activation dtype, the last rd columns of every head rotated in pairs
+// q float32 [T, heads (dim + rd)] -> the activation dtype, the last rd columns of every head rotated
 template <typename TA>
 __global__ void __launch_bounds__(256)
 latent_q_rope_kernel(const float* __restrict__ q, int ld, const int32_t* __restrict__ positions,
-                     const float* __restrict__ freq, int rot, TA* __restrict__ out, int heads, int dim, int rd) {
+                     const float* __restrict__ freq, int rot, int interleaved, TA* __restrict__ out, int heads,
+                     int dim, int rd) {
   __shared__ float cs[128], sn[128];
   const int t = blockIdx.x;
   angles(positions[t], freq, rot, 1.0f, cs, sn);
@@ -141,7 +143,7 @@ latent_q_rope_kernel(const float* __restrict__ q, int ld, const int32_t* __restr
   for (int i = threadIdx.x; i < heads * hw; i += 256) {
     const int h = i / hw, d = i % hw;
     float v = p[i];
-    if (d >= dim && d - dim < rot) v = turned(p + h * hw + dim, d - dim, rot, 1, cs, sn);
+    if (d >= dim && d - dim < rot) v = turned(p + h * hw + dim, d - dim, rot, interleaved, cs, sn);
     out[(size_t)t * heads * hw + i] = from_f32<TA>(v);
   }
 }
@@ -189,19 +191,19 @@ extern "C" int atoma_tied_rope_prepare(const float* proj, int ld, int off_q, int
 
 extern "C" int atoma_latent_rope_prepare(const float* proj, int ld, int off_dq, int off_c, int off_g, int q_rank,
                                          int rank, int rd, int rank_p, int n_gate, const float* wq, const float* wc,
-                                         float eps, const int32_t* positions, const float* freq, int rot, void* cq,
-                                         int act_dtype, void* kcache, void* vcache, int cache_dtype,
+                                         float eps, const int32_t* positions, const float* freq, int rot, int interleaved,
+                                         void* cq, int act_dtype, void* kcache, void* vcache, int cache_dtype,
                                          const int32_t* slot_mapping, int page_size, float* gate, int n_tokens,
                                          hipStream_t stream) {
   if (n_tokens <= 0) return 0;
-  if (q_rank <= 0 || rank <= 0 || rd < 0 || rank_p < rank + rd || n_gate <= 0 || rot < 0 || rot % 2 || rot > rd ||
+  if (q_rank <= 0 || rank <= 0 || rd < 0 || rank_p < rank + rd || n_gate < 0 || rot < 0 || rot % 2 || rot > rd ||
       rot > 256 || page_size <= 0 || off_dq < 0 || off_c < 0 || off_g < 0 || ld < off_dq + q_rank ||
       ld < off_c + rank + rd || ld < off_g + n_gate)
     return ATOMA_ERR_SHAPE;
 #define ATOMA_LRP(TA, TC)                                                                                            \
   hipLaunchKernelGGL((latent_rope_prepare_kernel<TA, TC>), dim3(n_tokens), dim3(256), 0, stream, proj, ld, off_dq,   \
-                     off_c, off_g, q_rank, rank, rd, rank_p, n_gate, wq, wc, eps, positions, freq, rot, (TA*)cq,     \
-                     (TC*)kcache, (TC*)vcache, slot_mapping, page_size, gate)
+                     off_c, off_g, q_rank, rank, rd, rank_p, n_gate, wq, wc, eps, positions, freq, rot, interleaved, \
+                     (TA*)cq, (TC*)kcache, (TC*)vcache, slot_mapping, page_size, gate)
   if (act_dtype == kF32 && cache_dtype == kF32) ATOMA_LRP(float, float);
   else if (act_dtype == kBF16 && cache_dtype == kBF16) ATOMA_LRP(bf16_t, bf16_t);
   else return ATOMA_ERR_DTYPE;
@@ -211,7 +213,7 @@ extern "C" int atoma_latent_rope_prepare(const float* proj, int ld, int off_dq, 
 }
 
 extern "C" int atoma_latent_q_rope(const float* q, int ld, const int32_t* positions, const float* freq, int rot,
-                                   void* out, int out_dtype, int n_tokens, int heads, int dim, int rd,
+                                   int interleaved, void* out, int out_dtype, int n_tokens, int heads, int dim, int rd,
                                    hipStream_t stream) {
   if (n_tokens <= 0) return 0;
   if (heads <= 0 || dim < 0 || rd < 0 || dim + rd <= 0 || rot < 0 || rot % 2 || rot > rd || rot > 256 ||
@@ -219,10 +221,10 @@ extern "C" int atoma_latent_q_rope(const float* q, int ld, const int32_t* positi
     return ATOMA_ERR_SHAPE;
   if (out_dtype == kF32)
     hipLaunchKernelGGL((latent_q_rope_kernel<float>), dim3(n_tokens), dim3(256), 0, stream, q, ld, positions, freq,
-                       rot, (float*)out, heads, dim, rd);
+                       rot, interleaved, (float*)out, heads, dim, rd);
   else if (out_dtype == kBF16)
     hipLaunchKernelGGL((latent_q_rope_kernel<bf16_t>), dim3(n_tokens), dim3(256), 0, stream, q, ld, positions, freq,
-                       rot, (bf16_t*)out, heads, dim, rd);
+                       rot, interleaved, (bf16_t*)out, heads, dim, rd);
   else
     return ATOMA_ERR_DTYPE;
   ATOMA_LAUNCH_CHECK();

@@ -60,7 +60,17 @@ HIP_MODULES: Dict[str, Tuple[Sequence[str], Sequence[str]]] = {
     "gated_attention": (("gated_attention.hip",), ()),
     "lightning": (("lightning.hip",), ()),
     "rglru": (("rglru.hip",), ()),
+    "linear_attention": (("linear_attention.hip",), ()),
 }
+
+# ... and once per padded key size that a model with such a mechanism has
+LINEAR_ATTENTION_SIZES = tuple(range(32, 257, 32))
+
+
+def linear_attention_module(padded_dim: int) -> Tuple[str, Sequence[str], Sequence[str]]:
+    """(name, sources, definitions) of the chunked linear-attention kernels for key sizes padded to ``padded_dim``."""
+    return f"linear_attention_d{padded_dim}", ("linear_attention_chunks.hip",), (f"ATOMA_LA_DP={padded_dim}",)
+
 
 _loaded: Dict[str, ctypes.CDLL] = {}
 _lock = threading.Lock()
@@ -232,6 +242,7 @@ def build_all(head_sizes: Sequence[int] = STANDARD_HEAD_SIZES) -> List[str]:
              for hd in head_sizes]
     jobs += [(attention_bf16.module_name(hd, page), ("attention_mfma.hip",), attention_bf16.module_defines(hd, page))
              for hd, page in LARGER_PAGE_MODULES]
+    jobs += [linear_attention_module(dp) for dp in LINEAR_ATTENTION_SIZES]
     with ThreadPoolExecutor(min(8, len(jobs))) as pool:
         futs = [pool.submit(load_hip_module, n, src, d, force_build=True) for n, src, d in jobs]
         for (n, _, _), f in zip(jobs, futs):

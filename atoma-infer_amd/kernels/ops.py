@@ -8,11 +8,12 @@ library raises ``KernelBuildError``; there is no other code path.
 from __future__ import annotations
 
 import ctypes
+import dataclasses
 from typing import Optional
 
 import torch
 
-from .library import load_hip_module
+from .library import linear_attention_module, load_hip_module
 
 F32, BF16 = 0, 1
 _CODES = {torch.float32: F32, torch.bfloat16: BF16}
@@ -84,8 +85,9 @@ def core():
 
 # ------------------------------------------------------------------------------------------------------------
 
-def embed(tokens: torch.Tensor, table: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """out[t] = table[tokens[t]] as float32; a token outside the table gives a row of NaN."""
+def embed(tokens: torch.Tensor, table: torch.Tensor, out: Optional[torch.Tensor] = None,
+          scale: float = 1.0) -> torch.Tensor:
+    """out[t] = table[tokens[t]] * scale as float32; a token outside the table gives a row of NaN."""
     _dev(tokens, table)
     _i32(tokens, "tokens")
     _need(table.dim() == 2 and table.is_contiguous(), "embedding table must be contiguous [vocab, width]")
@@ -94,12 +96,12 @@ def embed(tokens: torch.Tensor, table: torch.Tensor, out: Optional[torch.Tensor]
         out = torch.empty((n, width), dtype=torch.float32, device=table.device)
     _need(out.dtype is torch.float32 and out.is_contiguous() and tuple(out.shape) == (n, width), "embed: bad out")
     _check(core().atoma_embed(_p(tokens), _p(table), _code(table, "embedding table"), _p(out), n, width,
-                              table.shape[0], _stream()), "embed")
+                              table.shape[0], ctypes.c_float(scale), _stream()), "embed")
     return out
 
 
-def embed_begin_norm(tokens: torch.Tensor, table: torch.Tensor, gamma: torch.Tensor):
-    """The embedding gather with a norm begun, for at most 16 tokens: (resid float32 [T, W], u bfloat16 [T, W] =
+def embed_begin_norm(tokens: torch.Tensor, table: torch.Tensor, gamma: torch.Tensor, scale: float = 1.0):
+    """The embedding gather (rows times ``scale``) with a norm begun, for at most 16 tokens: (resid float32 [T, W], u bfloat16 [T, W] =
     resid * gamma, ss float32 [1, 16] the rows' sums of squares).  A product finishes the norm (gemm_bf16)."""
     _dev(tokens, table, gamma)
     _i32(tokens, "tokens")
@@ -112,7 +114,7 @@ def embed_begin_norm(tokens: torch.Tensor, table: torch.Tensor, gamma: torch.Ten
     ss = torch.empty((1, 16), dtype=torch.float32, device=table.device)
     _check(core().atoma_embed_begin_norm(_p(tokens), _p(table), _code(table, "embedding table"), _p(resid), _p(gamma),
                                          _code(gamma, "norm weight"), _p(u), _p(ss), n, width, table.shape[0],
-                                         _stream()), "embed_begin_norm")
+                                         ctypes.c_float(scale), _stream()), "embed_begin_norm")
     return resid, u, ss
 
 
@@ -240,11 +242,29 @@ def paged_attention_generic(q: torch.Tensor, kcache: torch.Tensor, vcache: torch
         page_size, t, nh, nkv, hd, _p(slopes), int(chunk), _p(sinks), _stream()), "paged_attention_generic")
 
 
-GATE_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1}
+GATE_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1, "relu": 2, "clamped_sigmoid": 3}
 
 
-def swiglu(gu: torch.Tensor, out: Optional[torch.Tensor] = None, block: int = 0, act: str = "silu") -> torch.Tensor:
-    """out[t, i] = act(gate[t, i]) * up[t, i] for gu [T, 2 I]; ``act``: "silu", or "gelu_tanh" (gelu's tanh form).
+def gate_activation(act) -> tuple:
+    """(kind, limit, slope) as the kernels take them, for "silu", "gelu_tanh", "relu" (act(gate) * up) or
+    ("clamped_sigmoid", limit, slope): g sigmoid(slope g) (u + 1) with g = min(gate, limit) and u = up held between
+    -limit and limit."""
+    name, *consts = (act,) if isinstance(act, str) else tuple(act)
+    if name not in GATE_ACTIVATIONS or len(consts) != (2 if name == "clamped_sigmoid" else 0) \
+            or (consts and not float(consts[0]) > 0):
+        raise ValueError(f"gate activation {act!r} is not supported (known: {', '.join(GATE_ACTIVATIONS)}; "
+                         f"'clamped_sigmoid' comes with a positive limit and a slope)")
+    limit, slope = (float(c) for c in consts) if consts else (0.0, 0.0)
+    return GATE_ACTIVATIONS[name], limit, slope
+
+
+def _gate_args(act):
+    kind, limit, slope = gate_activation(act)
+    return kind, ctypes.c_float(limit), ctypes.c_float(slope)
+
+
+def swiglu(gu: torch.Tensor, out: Optional[torch.Tensor] = None, block: int = 0, act="silu") -> torch.Tensor:
+    """out[t, i] = act(gate[t, i]) * up[t, i] for gu [T, 2 I]; ``act``: as ``gate_activation`` takes it.
 
     ``block`` 0: gate is the first half of a row and up the second; 16: blocks of 16 gate values followed by
     their 16 up values (the order of the fused gate-up product's weight rows).
@@ -256,7 +276,7 @@ def swiglu(gu: torch.Tensor, out: Optional[torch.Tensor] = None, block: int = 0,
         out = torch.empty((t, inter), dtype=gu.dtype, device=gu.device)
     _need(out.is_contiguous() and tuple(out.shape) == (t, inter) and out.dtype is gu.dtype, "swiglu: bad out")
     _check(core().atoma_swiglu(_p(gu), _p(out), _code(gu, "swiglu input"), t, inter, int(block),
-                               GATE_ACTIVATIONS[act], _stream()), "swiglu")
+                               *_gate_args(act), _stream()), "swiglu")
     return out
 
 
@@ -654,13 +674,20 @@ def head_linear(x: torch.Tensor, w: torch.Tensor, out_dtype: torch.dtype, gate: 
 
 
 
+ROUTER_SCORES = {"sigmoid": 0, "softmax": 1, "softmax_chosen": 2}
+
+
 def route_topk(logits: torch.Tensor, top: int, score: str = "sigmoid", correction: Optional[torch.Tensor] = None,
-               scale: float = 1.0):
+               scale: float = 1.0, bias: Optional[torch.Tensor] = None):
     """(ids int32 [T, top], weights float32 [T, top]).  Scores are sigmoid(logits) or ("softmax") the softmax of a
     row; the ``top`` experts with the largest score + ``correction`` [experts] are chosen and weighed by
-    score * ``scale``."""
-    _dev(logits, correction)
-    _need(score in ("sigmoid", "softmax"), "route_topk: scores are 'sigmoid' or 'softmax'")
+    score * ``scale``.  "softmax_chosen": the largest logits are chosen and weighed by the softmax over the chosen
+    ones, times ``scale``.  ``bias`` [experts] joins the logits first."""
+    _dev(logits, correction, bias)
+    _need(score in ROUTER_SCORES, f"route_topk: scores are one of {', '.join(ROUTER_SCORES)}")
+    _need(score != "softmax_chosen" or correction is None, "route_topk: a correction needs scores of its own")
+    if bias is not None:
+        _f32(bias, "bias", logits.shape[1])
     if correction is not None:
         _f32(correction, "correction", logits.shape[1])
     _need(logits.dtype is torch.float32 and logits.dim() == 2 and logits.stride(1) == 1, "router logits: float32 [T, E]")
@@ -668,7 +695,7 @@ def route_topk(logits: torch.Tensor, top: int, score: str = "sigmoid", correctio
     ids = torch.empty((t, top), dtype=torch.int32, device=logits.device)
     scores = torch.empty((t, top), dtype=torch.float32, device=logits.device)
     _check(_module("experts").atoma_route_topk(_p(logits), logits.stride(0), e, int(top), _p(ids), _p(scores), t,
-                                               1 if score == "softmax" else 0, _p(correction), ctypes.c_float(scale),
+                                               ROUTER_SCORES[score], _p(correction), ctypes.c_float(scale), _p(bias),
                                                _stream()), "route_topk")
     return ids, scores
 
@@ -734,10 +761,10 @@ def expert_gemm_mfma_ok(n: int, k: int) -> bool:
 
 def expert_gemm_mfma(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, perm, offsets, tiles, top: int, *,
                      swiglu: bool = False, planes: bool = False, tile_m: int = 64, relu2: bool = False,
-                     out_scale: Optional[torch.Tensor] = None) -> None:
+                     out_scale: Optional[torch.Tensor] = None, act="silu") -> None:
     """The grouped product on the matrix cores: a bfloat16 [places, K] in the order of ``perm``, w bfloat16
     [experts, N, K].  ``swiglu``: w's rows in blocks of 16 gate rows and their 16 up rows, out bfloat16
-    [places, N / 2] = silu(gate) * up; ``relu2``: out bfloat16 [places, N], the result's positive part squared; else out
+    [places, N / 2] = silu(gate) * up, or what ``act`` (``gate_activation``) makes of the two; ``relu2``: out bfloat16 [places, N], the result's positive part squared; else out
     float32 [places, N] or, with ``planes``, [top, T, N] by slot, times ``out_scale`` [slots] where given.
     ``tile_m``: what ``route_group`` was told."""
     _dev(a, w, out, perm, offsets, tiles, out_scale)
@@ -755,8 +782,8 @@ def expert_gemm_mfma(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, perm, 
     _need(offsets.numel() == e + 1 and tiles.dim() == 2 and tiles.shape[1] == 2, "expert_gemm_mfma: bad grouping")
     _check(_module("experts").atoma_expert_gemm_mfma(
         _p(a), _p(w), _p(out), cols, n, k, _p(perm), _p(offsets), _p(tiles), tiles.shape[0], int(top),
-        n_slots // top if planes else 0, 1 if swiglu else 2 if relu2 else 0, int(tile_m), _p(out_scale), _stream()),
-        "expert_gemm_mfma")
+        n_slots // top if planes else 0, 1 if swiglu else 2 if relu2 else 0, int(tile_m), _p(out_scale),
+        *_gate_args(act), _stream()), "expert_gemm_mfma")
 
 
 def relu2_gate(u: torch.Tensor, ff: int, off_gate: int, out_dtype: torch.dtype) -> torch.Tensor:
@@ -1061,10 +1088,13 @@ def tied_rope_prepare(proj: torch.Tensor, offsets, bq, bk, positions, freq: torc
 
 def latent_rope_prepare(proj: torch.Tensor, offsets, q_rank: int, rank: int, rd: int, rank_p: int, n_gate: int,
                         wq: torch.Tensor, wc: torch.Tensor, eps: float, positions, freq: torch.Tensor, rot: int,
-                        kcache, vcache, slot_mapping, page_size: int, act_dtype: torch.dtype):
+                        kcache, vcache, slot_mapping, page_size: int, act_dtype: torch.dtype,
+                        interleaved: bool = True):
     """(cq [T, q_rank] in ``act_dtype``, gate float32 [T, n_gate] = sigmoid) from ``proj`` float32 [T, ld] whose columns
     ``offsets`` = (query latent, key/value latent followed by the rotated key part, gates) name; the cache tiles
-    receive [c | rotated part | 0] as the key and [c | 0] as the value, ``rank_p`` columns each."""
+    receive [c | rotated part | 0] as the key and [c | 0] as the value, ``rank_p`` columns each.  ``n_gate`` 0:
+    no gates, and the second result is None.  Pairs (2i, 2i + 1) are rotated, or (i, i + rot / 2) if not
+    ``interleaved``."""
     _dev(proj, wq, wc, positions, freq, kcache, vcache, slot_mapping)
     t = proj.shape[0]
     off_dq, off_c, off_g = (int(o) for o in offsets)
@@ -1079,18 +1109,18 @@ def latent_rope_prepare(proj: torch.Tensor, offsets, q_rank: int, rank: int, rd:
     _tiles_ok(kcache, vcache, 1, page_size, rank_p)
     _need(kcache.dtype is act_dtype, "the cache must be of the activation dtype")
     cq = torch.empty((t, q_rank), dtype=act_dtype, device=proj.device)
-    gate = torch.empty((t, n_gate), dtype=torch.float32, device=proj.device)
+    gate = torch.empty((t, n_gate), dtype=torch.float32, device=proj.device) if n_gate else None
     _check(_module("gated_attention").atoma_latent_rope_prepare(
         _p(proj), proj.stride(0), off_dq, off_c, off_g, q_rank, rank, rd, rank_p, n_gate, _p(wq), _p(wc),
-        ctypes.c_float(eps), _p(positions), _p(freq), int(rot), _p(cq), _code(cq, "cq"), _p(kcache), _p(vcache),
+        ctypes.c_float(eps), _p(positions), _p(freq), int(rot), int(bool(interleaved)), _p(cq), _code(cq, "cq"), _p(kcache), _p(vcache),
         _code(kcache, "cache"), _p(slot_mapping), int(page_size), _p(gate), t, _stream()), "latent_rope_prepare")
     return cq, gate
 
 
 def latent_q_rope(q: torch.Tensor, positions, freq: torch.Tensor, rot: int, heads: int, dim: int, rd: int,
-                  out_dtype: torch.dtype) -> torch.Tensor:
+                  out_dtype: torch.dtype, interleaved: bool = True) -> torch.Tensor:
     """q float32 [T, heads (dim + rd)] in ``out_dtype`` with the first ``rot`` of every head's last ``rd`` columns
-    rotated in neighbouring pairs."""
+    rotated in neighbouring pairs, or in pairs (i, i + rot / 2) if not ``interleaved``."""
     _dev(q, positions, freq)
     t = q.shape[0]
     _need(q.dtype is torch.float32 and q.dim() == 2 and q.stride(1) == 1 and q.shape[1] >= heads * (dim + rd),
@@ -1098,7 +1128,7 @@ def latent_q_rope(q: torch.Tensor, positions, freq: torch.Tensor, rot: int, head
     _i32(positions, "positions", t)
     _f32(freq, "frequencies", rot // 2)
     out = torch.empty((t, heads * (dim + rd)), dtype=out_dtype, device=q.device)
-    _check(_module("gated_attention").atoma_latent_q_rope(_p(q), q.stride(0), _p(positions), _p(freq), int(rot), _p(out),
+    _check(_module("gated_attention").atoma_latent_q_rope(_p(q), q.stride(0), _p(positions), _p(freq), int(rot), int(bool(interleaved)), _p(out),
                                                           _code(out, "out"), t, heads, dim, rd, _stream()),
            "latent_q_rope")
     return out
@@ -1160,6 +1190,123 @@ def lightning_out(o: torch.Tensor, proj: torch.Tensor, off_g: int, w: torch.Tens
     _check(_module("lightning").atoma_lightning_out(_p(o), _p(proj), proj.stride(0) if t > 1 else proj.shape[1],
                                                     int(off_g), _p(w), ctypes.c_float(eps), _p(y), _code(y, "y"), t, n,
                                                     _stream()), "lightning_out")
+    return y
+
+
+@dataclasses.dataclass(frozen=True)
+class LinearAttentionSizes:
+    """Sizes and constants of a linear attention with a decaying state (linear_attention.h): ``offsets`` = the columns of
+    q, k, v and the gates in the projection; ``low`` = (column, number) of the low-rank values that the decays are made
+    of, None where the decays are fixed; ``rot`` columns of q and k are rotated."""
+    heads: int
+    dim: int
+    vdim: int
+    offsets: tuple
+    eps: float
+    q_scale: float = 1.0
+    k_scale: float = 1.0
+    rot: int = 0
+    low: Optional[tuple] = None
+    inv_tau: float = 1.0
+
+
+@dataclasses.dataclass(frozen=True)
+class LinearAttentionTensors:
+    """Its tensors, float32: ``decay`` [heads], or ``w2`` [heads dim, rank] and ``b2`` [heads dim]; ``freq`` [rot / 2];
+    ``norm`` [vdim] or None."""
+    decay: Optional[torch.Tensor] = None
+    w2: Optional[torch.Tensor] = None
+    b2: Optional[torch.Tensor] = None
+    freq: Optional[torch.Tensor] = None
+    norm: Optional[torch.Tensor] = None
+
+
+LINEAR_ATTENTION_CHUNK = 64
+LINEAR_ATTENTION_CHUNKED_MAX_VDIM = 512
+
+
+def linear_attention_plan(counts, chunked_from: int):
+    """The chunks of a step for ``linear_attention``: (int32 array, (chunks, entries cut into chunks, tokens of the
+    longest entry that is not)).  The array holds a row (entry, first token, tokens, 0) per chunk, then a row (entry,
+    first chunk, chunks, 0) per entry of at least ``chunked_from`` tokens (0: no entry is cut).  A function of the
+    entries' lengths."""
+    import numpy as np
+    rows, entries, t0, short = [], [], 0, 0
+    for e, c in enumerate(int(c) for c in counts):
+        if chunked_from and c >= chunked_from:
+            entries.append((e, len(rows), -(-c // LINEAR_ATTENTION_CHUNK), 0))
+            rows += [(e, t0 + lo, min(LINEAR_ATTENTION_CHUNK, c - lo), 0) for lo in range(0, c, LINEAR_ATTENTION_CHUNK)]
+        else:
+            short = max(short, c)
+        t0 += c
+    return np.asarray(rows + entries, dtype=np.int32).reshape(-1), (len(rows), len(entries), short)
+
+
+def linear_attention(proj: torch.Tensor, sizes: LinearAttentionSizes, w: LinearAttentionTensors, positions, q_start,
+                     state_slots, state: torch.Tensor, out_dtype: torch.dtype, plan, chunked_from: int) -> torch.Tensor:
+    """y [T, heads vdim] in ``out_dtype`` from ``proj`` float32 [T, ld]: the recurrence over every entry's tokens from and
+    into the requests' rows of ``state`` float32 [slots, heads vdim dim], its result normed head by head and gated.
+    ``plan``: (int32 device tensor, meta) of ``linear_attention_plan`` for the same ``chunked_from``, None only if that is
+    0; entries cut into chunks need ``out_dtype`` bfloat16."""
+    _dev(proj, positions, q_start, state_slots, state, w.decay, w.w2, w.b2, w.freq, w.norm)
+    t, n_entries = proj.shape[0], state_slots.numel()
+    h, dim, vdim = sizes.heads, sizes.dim, sizes.vdim
+    _need(proj.dtype is torch.float32 and proj.dim() == 2 and proj.stride(1) == 1, "proj must be float32 [T, ld]")
+    ends = [o + h * (dim if i < 2 else vdim) for i, o in enumerate(sizes.offsets)]
+    _need(min(sizes.offsets) >= 0 and max(ends) <= proj.shape[1], "the projections' columns do not fit proj")
+    _need(0 < dim <= 256, "linear_attention: key sizes beyond 256 are not supported")
+    _i32(q_start, "q_start", n_entries + 1)
+    _i32(state_slots, "state_slots")
+    _need(state.dtype is torch.float32 and state.is_contiguous() and state.dim() == 2
+          and state.shape[1] == h * vdim * dim, "the state must be float32 [slots, heads * vdim * dim]")
+    if w.decay is not None:
+        _f32(w.decay, "decay", h)
+        _need(sizes.low is None, "decays are fixed or made of low-rank values, not both")
+    else:
+        off, rank = sizes.low
+        _need(sizes.rot == 0 and rank > 0 and off >= 0 and off + rank <= proj.shape[1],
+              "the low-rank columns do not fit proj")
+        _f32(w.w2, "w2", h * dim * rank)
+        _f32(w.b2, "b2", h * dim)
+    if sizes.rot:
+        _need(sizes.rot % 2 == 0 and 0 < sizes.rot <= dim, "linear_attention: bad number of rotated columns")
+        _i32(positions, "positions", t)
+        _f32(w.freq, "frequencies", sizes.rot // 2)
+    if w.norm is not None:
+        _f32(w.norm, "norm weight", vdim)
+    y = torch.empty((t, h * vdim), dtype=out_dtype, device=proj.device)
+    low = sizes.low or (0, 0)
+    ld = proj.stride(0) if t > 1 else proj.shape[1]
+    at = (ctypes.c_int32 * 7)(ld, *(int(o) for o in sizes.offsets), int(low[0]), int(low[1]))
+    args = (_p(proj), at, _p(w.decay), _p(w.w2), _p(w.b2), ctypes.c_float(sizes.inv_tau), _p(positions), _p(w.freq),
+            int(sizes.rot), ctypes.c_float(sizes.q_scale), ctypes.c_float(sizes.k_scale), _p(w.norm),
+            ctypes.c_float(sizes.eps), _p(q_start), _p(state_slots), _p(state), h, dim, vdim)
+    n_chunks, n_long, short = (0, 0, None)
+    if chunked_from:
+        arr, (n_chunks, n_long, short) = plan
+        _i32(arr, "chunks", 4 * (n_chunks + n_long))
+    if short != 0:
+        lib = _module("linear_attention")
+        # tokens that pass LDS at a time: as many as the longest entry has, up to 16
+        tb = 16 if short is None else next(b for b in (1, 2, 4, 8, 16) if b >= min(short, 16))
+        o = torch.empty((t, h * vdim), dtype=torch.float32, device=proj.device) \
+            if lib.atoma_linear_attention_needs_o(dim, vdim) else None
+        _check(lib.atoma_linear_attention_scan(*args, _p(y), _code(y, "y"), _p(o), n_entries, tb,
+                                               int(chunked_from), _stream()), "linear_attention_scan")
+    if n_chunks:
+        _need(out_dtype is torch.bfloat16 and vdim <= LINEAR_ATTENTION_CHUNKED_MAX_VDIM,
+              "linear_attention: chunks leave bfloat16, and up to 512 value columns a head")
+        dp, vp = -(-dim // 32) * 32, -(-vdim // 16) * 16
+        lib = load_hip_module(*linear_attention_module(dp))
+        n = n_chunks * h
+        bf = dict(dtype=torch.bfloat16, device=proj.device)
+        f32 = dict(dtype=torch.float32, device=proj.device)
+        c = LINEAR_ATTENTION_CHUNK
+        wp, wq = torch.empty((n, 2, c, c), **bf), torch.empty((n, 2, c, dp), **bf)
+        wd, wu, ws = torch.empty((n, dp), **f32), torch.empty((n, vp, dp), **f32), torch.empty((n, 2, vp, dp), **bf)
+        _check(lib.atoma_linear_attention_chunked(
+            *args, _p(y), _p(arr), n_chunks, ctypes.c_void_p(arr.data_ptr() + 16 * n_chunks), n_long, _p(wp), _p(wq),
+            _p(wd), _p(wu), _p(ws), _stream()), "linear_attention_chunked")
     return y
 
 

@@ -13,7 +13,8 @@ from .linear import linear
 from .norm import RMSNorm
 from .parallel import ParallelMixer
 from .position import NoPosition, RotaryEncoding
-from .recurrent import GatedDeltaRule, GatedLinearRecurrence, LightningAttention, MinGRU, StateSpaceDuality
+from .recurrent import (DecayedLinearAttention, GatedDeltaRule, GatedLinearRecurrence, LightningAttention, MinGRU,
+                        StateSpaceDuality)
 from .streams import BigramEmbedding, StreamBlock, StreamsNorm, StreamUpdate
 
 __all__ = ["Block", "CacheSpec", "FeedForward", "Mixer", "Norm", "Part", "PositionEncoding", "StateSpec",
@@ -23,4 +24,4 @@ __all__ = ["Block", "CacheSpec", "FeedForward", "Mixer", "Norm", "Part", "Positi
            "SandwichBlock", "RoutedExperts", "ParallelMixer", "GatedDeltaRule", "LatentAttention", "SideBySideBlock",
            "LoopEntry", "NoMixer", "StateSpaceDuality", "DifferentialAttention", "MinGRU", "DepthAverage",
            "GatedTiedValueAttention", "RotaryLatentAttention", "DenseFeedForward", "GatedLinearRecurrence",
-           "LightningAttention", "BigramEmbedding", "StreamBlock", "StreamsNorm", "StreamUpdate"]
+           "LightningAttention", "DecayedLinearAttention", "BigramEmbedding", "StreamBlock", "StreamsNorm", "StreamUpdate"]

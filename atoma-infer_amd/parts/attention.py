@@ -24,6 +24,7 @@ import torch
 from ..kernels import ops
 from .base import CacheSpec, Mixer, PositionEncoding, WeightSpec, register_mixer
 from .linear import as_tensor, linear, linear_delta
+from .position import rotation_frequencies
 
 
 class PagedAttention(Mixer):
@@ -489,29 +490,6 @@ class DifferentialAttention(PagedAttention):
         return linear_delta(y, self.w_o, None, self.w_o_tiled)
 
 
-def rotation_frequencies(base: float, dims: int, scaling: Optional[dict] = None):
-    """(float32 tensor [dims / 2] of base^(-2i / dims), worked out in double precision and rounded once; the factor on
-    cosines and sines).  ``scaling`` = {factor, original, fast, slow} slows the long waves down: with
-    where(t) = dims ln(original / (2 pi t)) / (2 ln base), lo = max(floor(where(fast)), 0), hi = min(ceil(where(slow)),
-    dims - 1) and ramp_i = clamp((i - lo) / max(hi - lo, 0.001), 0, 1), pair i turns at
-    f_i / factor * ramp_i + f_i (1 - ramp_i), and cosines and sines are multiplied by 0.1 ln(factor) + 1."""
-    i = torch.arange(dims // 2, dtype=torch.float64)
-    f = torch.pow(torch.tensor(float(base), dtype=torch.float64), -2.0 * i / max(dims, 1))
-    mag = 1.0
-    if scaling is not None:
-        factor, original = float(scaling["factor"]), float(scaling["original"])
-
-        def where(turns: float) -> float:
-            return dims * math.log(original / (2.0 * math.pi * turns)) / (2.0 * math.log(base))
-
-        lo = max(math.floor(where(float(scaling["fast"]))), 0)
-        hi = min(math.ceil(where(float(scaling["slow"]))), dims - 1)
-        ramp = torch.clamp((i - lo) / max(hi - lo, 0.001), 0.0, 1.0)
-        f = f / factor * ramp + f * (1.0 - ramp)
-        mag = 0.1 * math.log(factor) + 1.0
-    return f.to(torch.float32), mag
-
-
 class GatedTiedValueAttention(PagedAttention):
     """Attention whose values are its keys as projected (with their bias, before the rotation; no value projection),
     with an output gate per column:
@@ -611,9 +589,11 @@ class RotaryLatentAttention(PagedAttention):
       the latent c; the rest, rotated, is a key part of its own.  Per head k = [W_uk c | that part], v = W_uv c
       (``value_size`` columns); the cache keeps c and the rotated part, nothing else;
     * rotation of neighbouring pairs (2i, 2i + 1) of the first ``rotary_dim`` of the ``rotary_size`` columns by
-      position * base^(-2i / rotary_dim), angles in float32 from the position;
-    * every earlier key is seen, ordinary softmax, the scale given; the heads' outputs are multiplied column by column
-      with sigmoid(W_g x), then W_o.
+      position * base^(-2i / rotary_dim), angles in float32 from the position; with ``interleaved`` False the pairs
+      are (i, i + rotary_dim / 2);
+    * every earlier key is seen, or with ``window`` the last ``window`` of them (the token's own included), ordinary
+      softmax, the scale given; with ``gated`` the heads' outputs are multiplied column by column with sigmoid(W_g x);
+      then W_o.
 
     As in ``LatentAttention`` the heads' key and value maps act on the query's side: the attention kernels run with
     one shared key head [c | rotated part] of ``rank + rotary_size`` columns (rounded up to a multiple of 16) against
@@ -621,15 +601,17 @@ class RotaryLatentAttention(PagedAttention):
 
     Tensors ([out, in]): ``dq`` [q_rank, width], ``dq.norm``, ``uq`` [heads (head_size + rotary_size), q_rank], ``dkv``
     [rank + rotary_size, width], ``dkv.norm`` [rank], ``uk`` [heads head_size, rank], ``uv`` [heads value_size, rank],
-    ``g`` [heads value_size, width], ``o`` [width, heads value_size].
+    ``g`` [heads value_size, width] (if ``gated``), ``o`` [width, heads value_size].
     """
 
     def __init__(self, width: int, num_heads: int, head_size: int, rotary_size: int, value_size: int, rank: int,
                  q_rank: int, scale: float, norm_eps: float, rotary_base: float = 10000.0,
-                 rotary_dim: Optional[int] = None):
+                 rotary_dim: Optional[int] = None, interleaved: bool = True, gated: bool = True,
+                 window: Optional[int] = None):
         wide = -(-(int(rank) + int(rotary_size)) // 16) * 16
-        super().__init__(width, num_heads, 1, wide, None, None, scale, None)
-        self.qd, self.rd, self.vd, self.rank, self.q_rank = int(head_size), int(rotary_size), int(value_size),             int(rank), int(q_rank)
+        super().__init__(width, num_heads, 1, wide, None, window, scale, None)
+        self.qd, self.rd, self.vd = int(head_size), int(rotary_size), int(value_size)
+        self.rank, self.q_rank, self.interleaved, self.gated = int(rank), int(q_rank), bool(interleaved), bool(gated)
         self.rot = self.rd if rotary_dim is None else int(rotary_dim)
         if self.rot % 2 or not 0 <= self.rot <= self.rd or self.rot > 256:
             raise ValueError(f"rotary_dim {self.rot} must be even, at most rotary_size {self.rd} and at most 256")
@@ -648,10 +630,10 @@ class RotaryLatentAttention(PagedAttention):
                 "uq": WeightSpec((h * (self.qd + self.rd), qr), std=qr ** -0.5),
                 "dkv": WeightSpec((r + self.rd, w)), "dkv.norm": WeightSpec((r,), "norm"),
                 "uk": WeightSpec((h * self.qd, r), std=r ** -0.5), "uv": WeightSpec((h * self.vd, r), std=r ** -0.5),
-                "g": WeightSpec((h * self.vd, w)), "o": WeightSpec((w, h * self.vd))}
+                **({"g": WeightSpec((h * self.vd, w))} if self.gated else {}), "o": WeightSpec((w, h * self.vd))}
 
     def load(self, get, device, act_dtype) -> None:
-        ws = [get("dq"), get("dkv"), get("g")]
+        ws = [get("dq"), get("dkv")] + ([get("g")] if self.gated else [])
         dt = ws[0].dtype if all(w.dtype is ws[0].dtype for w in ws) else torch.float32
         rows = sum(w.shape[0] for w in ws)
         parts = [w.to(device=device, dtype=dt) for w in ws]
@@ -691,15 +673,15 @@ class RotaryLatentAttention(PagedAttention):
         # both latents and the gates leave their product in float32: norms, rotation and gates are float32 work
         proj = linear(x, self.w_in, torch.float32)
         cq, gate = ops.latent_rope_prepare(proj, (0, self.off_c, self.off_g), self.q_rank, self.rank, self.rd, self.hd,
-                                           self.nh * self.vd, self.q_norm, self.c_norm, self.norm_eps, ctx.positions,
+                                           self.nh * self.vd if self.gated else 0, self.q_norm, self.c_norm, self.norm_eps, ctx.positions,
                                            self.freq, self.rot, cache.k, cache.v, cache.slot_mapping, cache.page_size,
-                                           x.dtype)
+                                           x.dtype, self.interleaved)
         q = ops.latent_q_rope(linear(cq, self.w_uq, torch.float32), ctx.positions, self.freq, self.rot, self.nh,
-                              self.qd, self.rd, x.dtype)
+                              self.qd, self.rd, x.dtype, self.interleaved)
         ql = ops.head_linear(q, self.w_uk, x.dtype)                      # the queries in the cached key's columns
         mixed = torch.empty((t, self.nh * self.hd), dtype=x.dtype, device=proj.device)
         self.attend(ql, cache.k, cache.v, mixed, ctx, cache)
-        out = ops.head_linear(mixed, self.w_uv, x.dtype, gate)           # the heads' values, gated column by column
+        out = ops.head_linear(mixed, self.w_uv, x.dtype, gate)           # the heads' values (gated column by column)
         return linear_delta(out, self.w_o, sink, self.w_o_tiled)
 
 

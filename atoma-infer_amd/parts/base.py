@@ -178,6 +178,10 @@ class Norm(Part):
         """(resid, Begun) for the rows ``table[tokens]`` with this norm begun; or None."""
         return None
 
+    def embed_scaled(self, table: torch.Tensor, tokens: torch.Tensor, scale: float):
+        """The same for the rows ``table[tokens] * scale``."""
+        return None
+
 
 class PositionEncoding(Part):
     """Encodes positions into queries and keys."""

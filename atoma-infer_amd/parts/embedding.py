@@ -16,8 +16,9 @@ from .linear import linear
 
 
 class TokenEmbedding(Part):
-    def __init__(self, vocab_size: int, width: int, name: str = "weight"):
-        self.vocab_size, self.width, self.name = int(vocab_size), int(width), str(name)
+    def __init__(self, vocab_size: int, width: int, name: str = "weight", scale: float = 1.0):
+        # ``scale`` multiplies the rows on their way into the stream; a head tied to the table reads it without
+        self.vocab_size, self.width, self.name, self.scale = int(vocab_size), int(width), str(name), float(scale)
         self.weight: Optional[torch.Tensor] = None
 
     def graph_safe(self) -> bool:
@@ -36,9 +37,11 @@ class TokenEmbedding(Part):
         """The float32 residual rows of ``tokens`` (into ``out`` where given); with ``norm`` (the norm that reads them
         first) a pair (rows, that norm begun or None)."""
         if norm is None:
-            return ops.embed(tokens, self.weight, out)
-        got = norm.embed(self.weight, tokens)
-        return got if got is not None else (ops.embed(tokens, self.weight), None)
+            return ops.embed(tokens, self.weight, out, self.scale)
+        # (a norm that cannot begin scaled rows is not asked to)
+        got = norm.embed(self.weight, tokens) if self.scale == 1.0 else \
+            norm.embed_scaled(self.weight, tokens, self.scale)
+        return got if got is not None else (ops.embed(tokens, self.weight, scale=self.scale), None)
 
 
 class OutputHead(Part):

@@ -1,5 +1,6 @@
 """Dense gated feed-forward: ``down(act(gate(x)) * up(x))``, no biases; act is SiLU (SwiGLU:
-models/src/llama.rs:362-366, 372-374) or, for designs that ask for it, the tanh form of GELU.
+models/src/llama.rs:362-366, 372-374) or, for designs that ask for it, the tanh form of GELU, relu, or a pair of clamped
+values (``kernels.ops.gate_activation``).
 
 gate and up are fused into one [2 I, width] matrix at load time, so one product feeds the SiLU-multiply kernel.
 When I is a multiple of 16 the rows are interleaved in blocks of 16 (16 gate rows, then the 16 up rows of the
@@ -19,12 +20,12 @@ from .linear import linear, linear_delta
 
 class SwiGLU(FeedForward):
     def __init__(self, width: int, intermediate: int,
-                 names=("gate_proj.weight", "up_proj.weight", "down_proj.weight"), activation: str = "silu"):
+                 names=("gate_proj.weight", "up_proj.weight", "down_proj.weight"), activation="silu"):
         # ``names``: the tensors of the gate, up and down matrices below the part's prefix
-        # ``activation``: of the gate, "silu" or "gelu_tanh" (0.5 g (1 + tanh(sqrt(2 / pi) (g + 0.044715 g^3))))
-        if activation not in ops.GATE_ACTIVATIONS:
-            raise ValueError(f"activation {activation!r} is not supported (known: {', '.join(ops.GATE_ACTIVATIONS)})")
-        self.activation = str(activation)
+        # ``activation``: how a gate value and an up value become one, as ``ops.gate_activation`` takes it: "silu",
+        # "gelu_tanh" (0.5 g (1 + tanh(sqrt(2 / pi) (g + 0.044715 g^3)))), "relu", ("clamped_sigmoid", limit, slope)
+        ops.gate_activation(activation)
+        self.activation = activation
         self.width, self.inter, self.names = int(width), int(intermediate), tuple(names)
         self.block = 0
         self.w_gate_up: Optional[torch.Tensor] = None

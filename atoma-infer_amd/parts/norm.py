@@ -87,9 +87,12 @@ class RMSNorm(Norm):
         return None
 
     def embed(self, table, tokens):
+        return self.embed_scaled(table, tokens, 1.0)
+
+    def embed_scaled(self, table, tokens, scale):
         if self.act_dtype is not torch.bfloat16 or tokens.numel() > 16 or table.shape[1] != self.width:
             return None
-        resid, u, ss = ops.embed_begin_norm(tokens, table, self.weight)
+        resid, u, ss = ops.embed_begin_norm(tokens, table, self.weight, scale)
         return resid, Begun(u, ss, self.eps, self.width, self)
 
 

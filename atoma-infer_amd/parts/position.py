@@ -98,5 +98,28 @@ def clear_tables() -> None:
     _TABLES.clear()
 
 
+def rotation_frequencies(base: float, dims: int, scaling: Optional[dict] = None):
+    """(float32 tensor [dims / 2] of base^(-2i / dims), worked out in double precision and rounded once; the factor on
+    cosines and sines).  ``scaling`` = {factor, original, fast, slow} slows the long waves down: with
+    where(t) = dims ln(original / (2 pi t)) / (2 ln base), lo = max(floor(where(fast)), 0), hi = min(ceil(where(slow)),
+    dims - 1) and ramp_i = clamp((i - lo) / max(hi - lo, 0.001), 0, 1), pair i turns at
+    f_i / factor * ramp_i + f_i (1 - ramp_i), and cosines and sines are multiplied by 0.1 ln(factor) + 1."""
+    i = torch.arange(dims // 2, dtype=torch.float64)
+    f = torch.pow(torch.tensor(float(base), dtype=torch.float64), -2.0 * i / max(dims, 1))
+    mag = 1.0
+    if scaling is not None:
+        factor, original = float(scaling["factor"]), float(scaling["original"])
+
+        def where(turns: float) -> float:
+            return dims * math.log(original / (2.0 * math.pi * turns)) / (2.0 * math.log(base))
+
+        lo = max(math.floor(where(float(scaling["fast"]))), 0)
+        hi = min(math.ceil(where(float(scaling["slow"]))), dims - 1)
+        ramp = torch.clamp((i - lo) / max(hi - lo, 0.001), 0.0, 1.0)
+        f = f / factor * ramp + f * (1.0 - ramp)
+        mag = 0.1 * math.log(factor) + 1.0
+    return f.to(torch.float32), mag
+
+
 register_position("rotary", RotaryEncoding)
 register_position("none", NoPosition)

@@ -30,6 +30,7 @@ import torch
 from ..kernels import ops
 from .base import FREE, Mixer, StateSpec, WeightSpec, register_mixer
 from .linear import linear, linear_delta
+from .position import rotation_frequencies
 
 
 class GatedDeltaRule(Mixer):
@@ -369,6 +370,137 @@ class LightningAttention(Mixer):
         return linear_delta(y, self.w_o, None, self.w_o_tiled)
 
 
+class DecayedLinearAttention(Mixer):
+    """Linear attention whose state decays, without softmax or denominator: q = W_q x, k = W_k x (``heads`` x ``dim``),
+    v = W_v x (``heads`` x ``vdim``); per head
+
+        S <- diag(alpha) S + k v^T;   o = S^T q;
+
+    o is RMS-normed over a head's ``vdim`` columns (``norm_weight``: plain weight ``norm`` [vdim], shared by the heads),
+    multiplied by silu(W_g x) and projected by W_o.  What differs between designs:
+
+    * the decay: one fixed number a head (``decay``), or a number per key channel and token (``tau``):
+      alpha = sigmoid(W_a2 (W_a1 x) + b)^(1 / tau), the inner size of the low-rank map being the checkpoint's;
+    * ``rotary_dim`` columns of every q and k head rotated, column i with column i + rotary_dim / 2, by
+      position * rotary_base^(-2i / rotary_dim), angles in float32 from the position;
+    * ``q_scale`` and ``k_scale``.
+
+    A request's state is S, float32 [heads][vdim][dim], zero at its start.  The input projections are one product with
+    float32 sums that leaves unrounded; rotation, decays, the recurrence, the norm and the gate are float32 in both
+    dtypes.  Decoded tokens and short entries are walked token by token, one kernel between the two projections.  With
+    bfloat16 activations, entries of ``CHUNKED_FROM`` tokens or more run in chunks of 64 tokens side by side on the
+    matrix cores (``ops.linear_attention_plan``, made once per step on the host), float32 operands in two bfloat16 terms
+    there and every sum float32.
+
+    Tensors ([out, in]): ``q``, ``k`` [heads dim, width], ``v``, ``g`` [heads vdim, width], ``o`` [width, heads vdim];
+    ``norm`` [vdim]; ``a1`` [rank, width], ``a2`` [heads dim, rank], ``a2.b`` [heads dim].
+    """
+
+    CHUNKED_FROM = 40
+
+    def __init__(self, width: int, heads: int, dim: int, vdim: int, norm_eps: float, decay=None,
+                 tau: Optional[float] = None, rank: Optional[int] = None, rotary_base: float = 10000.0,
+                 rotary_dim: int = 0, q_scale: float = 1.0, k_scale: float = 1.0, norm_weight: bool = False):
+        if (decay is None) == (tau is None):
+            raise ValueError("the decays are fixed (decay) or gated (tau), one of the two")
+        if decay is not None and (len(decay) != heads or any(not 0.0 <= float(d) <= 1.0 for d in decay)):
+            raise ValueError(f"{len(decay)} decays for {heads} heads; each lies between 0 and 1")
+        if tau is not None and (not float(tau) > 0 or rotary_dim):
+            raise ValueError("gated decays take a positive tau and no rotation")
+        if not 0 < dim <= 256 or vdim <= 0:
+            raise ValueError(f"key size {dim} is not supported: the recurrence's kernel takes up to 256")
+        if rotary_dim % 2 or not 0 <= rotary_dim <= dim:
+            raise ValueError(f"{rotary_dim} rotated columns must be even and fit the {dim} of a head")
+        self.width, self.heads, self.dim, self.vdim = int(width), int(heads), int(dim), int(vdim)
+        self.norm_eps, self.norm_weight = float(norm_eps), bool(norm_weight)
+        self.decay = None if decay is None else [float(d) for d in decay]
+        self.tau, self.rank = None if tau is None else float(tau), int(rank) if rank else None
+        self.rotary_base, self.rot = float(rotary_base), int(rotary_dim)
+        self.q_scale, self.k_scale = float(q_scale), float(k_scale)
+        self.w_in = self.w_in_tiled = self.w_o = self.w_o_tiled = self.sizes = self.tensors = None
+        self.chunked = 0
+
+    def graph_safe(self) -> bool:
+        return True     # entries, slots and lengths come from the step's device tensors, chunks from its plan
+
+    def weight_specs(self) -> Dict[str, WeightSpec]:
+        w, nq, nv = self.width, self.heads * self.dim, self.heads * self.vdim
+        specs = {"q": WeightSpec((nq, w), std=0.08), "k": WeightSpec((nq, w), std=0.08),
+                 "v": WeightSpec((nv, w), std=0.08), "g": WeightSpec((nv, w), std=0.08), "o": WeightSpec((w, nv))}
+        if self.norm_weight:
+            specs["norm"] = WeightSpec((self.vdim,), "norm")
+        if self.decay is None:
+            r = self.rank or FREE
+            specs.update({"a1": WeightSpec((r, w), std=0.1), "a2": WeightSpec((nq, r), std=0.3),
+                          "a2.b": WeightSpec((nq,), std=1.0, mean=1.0)})
+        return specs
+
+    def state_spec(self) -> StateSpec:
+        return StateSpec((self.heads * self.vdim * self.dim,), "float32")
+
+    def load(self, get, device, act_dtype) -> None:
+        nq, nv = self.heads * self.dim, self.heads * self.vdim
+        gated = self.decay is None
+        ws = [get(n) for n in ("q", "k", "v", "g")] + ([get("a1")] if gated else [])
+        dt = ws[0].dtype if all(w.dtype is ws[0].dtype for w in ws) else torch.float32
+        rows = sum(w.shape[0] for w in ws)
+        parts = [w.to(device=device, dtype=dt) for w in ws]
+        if (-rows) % 64:      # whole tiles for the matrix-core products
+            parts.append(torch.zeros(((-rows) % 64, self.width), dtype=dt, device=device))
+        self.w_in = torch.cat(parts, dim=0).contiguous()
+        self.w_o = get("o").to(device).contiguous()
+        f32 = dict(device=device, dtype=torch.float32)
+        low, w2, b2, decay = None, None, None, None
+        if gated:
+            self.rank = ws[4].shape[0]
+            w2, b2 = get("a2").to(**f32).contiguous(), get("a2.b").to(**f32).contiguous()
+            if w2.shape[1] != self.rank:
+                raise ValueError(f"the halves of the low-rank map do not fit: a1 {tuple(ws[4].shape)}, a2 {tuple(w2.shape)}")
+            low = (2 * nq + 2 * nv, self.rank)
+        else:
+            decay = torch.tensor(self.decay, dtype=torch.float64).to(**f32).contiguous()
+        freq = rotation_frequencies(self.rotary_base, self.rot)[0].to(device).contiguous() if self.rot else None
+        self.tensors = ops.LinearAttentionTensors(
+            decay, w2, b2, freq, get("norm").to(**f32).contiguous() if self.norm_weight else None)
+        self.sizes = ops.LinearAttentionSizes(self.heads, self.dim, self.vdim, (0, nq, 2 * nq, 2 * nq + nv), self.norm_eps,
+                                              self.q_scale, self.k_scale, self.rot, low,
+                                              1.0 / self.tau if gated else 1.0)
+        self.chunked = self.CHUNKED_FROM if act_dtype is torch.bfloat16 and \
+            self.vdim <= ops.LINEAR_ATTENTION_CHUNKED_MAX_VDIM else 0
+        self.w_in_tiled = self.w_o_tiled = None
+        if act_dtype is torch.bfloat16 and self.w_in.dtype is torch.bfloat16 and self.w_o.dtype is torch.bfloat16:
+            from ..kernels import gemm_bf16
+            plan = gemm_bf16.tiled_plan(self.w_in.shape[0], self.width, swiglu=False)
+            if plan is not None:
+                self.w_in_tiled = gemm_bf16.tile_weight(self.w_in, *plan)
+            self.w_o_tiled = gemm_bf16.tile_copies_resid(self.w_o)
+
+    def device_bytes(self) -> int:
+        t = self.tensors
+        return sum(w.numel() * w.element_size() for w in (self.w_in, self.w_o, t.w2) if w is not None)
+
+    def _plan_key(self):
+        return ("linear_attention_chunks", self.chunked)
+
+    def step_planner(self, page_size: int, cache_dtype: torch.dtype):
+        """(key, fn(starts, counts, bucket_tokens) -> (int32 array, meta)): the chunks of long entries."""
+        if not self.chunked:
+            return None
+        chunked = self.chunked
+        return self._plan_key(), lambda starts, counts, bucket: ops.linear_attention_plan(counts, chunked)
+
+    def forward(self, x, ctx, cache):
+        proj = linear(x, self.w_in, torch.float32, tiled=self.w_in_tiled)
+        plan = getattr(ctx, "plans", {}).get(self._plan_key())
+        if plan is None and self.chunked:
+            # a caller without a step planner (a test of the part alone): plan here and now
+            arr, meta = ops.linear_attention_plan(ctx.h_counts, self.chunked)
+            plan = (torch.from_numpy(arr).to(x.device), meta)
+        y = ops.linear_attention(proj, self.sizes, self.tensors, ctx.positions, ctx.q_start, ctx.state_slots, cache.state,
+                                 x.dtype, plan, self.chunked)
+        return linear_delta(y, self.w_o, None, self.w_o_tiled)
+
+
 class GatedLinearRecurrence(Mixer):
     """Griffin's recurrent block around a real-gated linear recurrent unit, ``inner`` channels:
 
@@ -469,5 +601,6 @@ class GatedLinearRecurrence(Mixer):
 register_mixer("gated_delta_rule", GatedDeltaRule)
 register_mixer("mingru", MinGRU)
 register_mixer("lightning_attention", LightningAttention)
+register_mixer("decayed_linear_attention", DecayedLinearAttention)
 register_mixer("gated_linear_recurrence", GatedLinearRecurrence)
 register_mixer("state_space_duality", StateSpaceDuality)
