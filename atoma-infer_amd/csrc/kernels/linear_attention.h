@@ -36,6 +36,7 @@ struct LinearAttention {
   float inv_tau;
   const int32_t* positions;     // [T], read if rot > 0
   const float* freq;            // [rot / 2]
+  const float* angles;          // [T, rot]: cosines, then sines of a token's pairs; read by the chunked kernels
   int rot;
   float q_scale, k_scale;
   const float* norm_w;          // [vdim] or null
@@ -59,9 +60,13 @@ __device__ __forceinline__ float row16_sum(float x) {
   return x;
 }
 
-// sigmoid(z)^(1 / tau) = exp(log sigmoid(z) / tau), log sigmoid(z) = min(z, 0) - log(1 + exp(-|z|))
+// sigmoid(z)^(1 / tau) = exp(log sigmoid(z) / tau), log sigmoid(z) = min(z, 0) - log(1 + exp(-|z|)).  The logarithm's
+// argument lies between 1 and 2, so its absolute error is that of a float near one, and with it the decay's relative
+// error; v_exp_f32 and v_log_f32 (base 2) are good to about one unit in the last place.
 __device__ __forceinline__ float gated_decay(float z, float inv_tau) {
-  return expf((fminf(z, 0.f) - log1pf(expf(-fabsf(z)))) * inv_tau);
+  constexpr float kLog2e = 1.4426950408889634f;
+  const float l = __builtin_amdgcn_logf(1.0f + __builtin_amdgcn_exp2f(-fabsf(z) * kLog2e));
+  return __builtin_amdgcn_exp2f((fminf(z, 0.f) * kLog2e - l) * inv_tau);
 }
 
 // column r of a head's rotated q or k; cs, sn: cosines and sines of the token's pairs
@@ -81,14 +86,15 @@ inline bool linear_attention_ok(const LinearAttention& a) {
   return a.rot == 0 || (a.positions && a.freq);
 }
 
-inline LinearAttention linear_attention_args(const float* proj, const int32_t* at, const float* decay, const float* w2, const float* b2,
-                            float inv_tau, const int32_t* positions, const float* freq, int rot, float q_scale,
-                            float k_scale, const float* norm_w, float eps, const int32_t* q_start,
-                            const int32_t* state_slots, float* state, int heads, int dim, int vdim) {
+inline LinearAttention linear_attention_args(const float* proj, const int32_t* at, const float* decay, const float* w2,
+                                            const float* b2, float inv_tau, const int32_t* positions, const float* freq,
+                                            const float* angles, int rot, float q_scale, float k_scale,
+                                            const float* norm_w, float eps, const int32_t* q_start,
+                                            const int32_t* state_slots, float* state, int heads, int dim, int vdim) {
   LinearAttention a;
   a.proj = proj, a.ld = at[0], a.off_q = at[1], a.off_k = at[2], a.off_v = at[3], a.off_g = at[4];
   a.decay = decay, a.off_low = at[5], a.rank = at[6], a.w2 = w2, a.b2 = b2, a.inv_tau = inv_tau;
-  a.positions = positions, a.freq = freq, a.rot = rot, a.q_scale = q_scale, a.k_scale = k_scale;
+  a.positions = positions, a.freq = freq, a.angles = angles, a.rot = rot, a.q_scale = q_scale, a.k_scale = k_scale;
   a.norm_w = norm_w, a.eps = eps, a.q_start = q_start, a.state_slots = state_slots, a.state = state;
   a.heads = heads, a.dim = dim, a.vdim = vdim;
   return a;

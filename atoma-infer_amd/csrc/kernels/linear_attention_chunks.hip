@@ -35,7 +35,7 @@ __device__ __forceinline__ uint16_t hi_of(float x) { return __builtin_bit_cast(u
 __device__ __forceinline__ uint16_t lo_of(float x, uint16_t hi) { return hi_of(x - bf16_bits_to_f32(hi)); }
 __device__ __forceinline__ bf16x8 frag(const uint16_t* p) { return *reinterpret_cast<const bf16x8*>(p); }
 __device__ __forceinline__ uint32_t pair(uint16_t a, uint16_t b) { return a | ((uint32_t)b << 16); }
-__device__ __forceinline__ float pow_int(float l2, int n) { return n == 0 ? 1.0f : exp2f(l2 * (float)n); }
+__device__ __forceinline__ float pow_int(float l2, int n) { return n == 0 ? 1.0f : __builtin_amdgcn_exp2f(l2 * (float)n); }
 
 // acc += A B with both operands in two terms
 __device__ __forceinline__ f32x4 mfma3(bf16x8 ah, bf16x8 al, bf16x8 bh, bf16x8 bl, f32x4 acc) {
@@ -55,21 +55,13 @@ __device__ __forceinline__ void scale_frag(bf16x8& fh, bf16x8& fl, const float* 
   }
 }
 
-// 16 values as two rows of bfloat16 terms
-__device__ __forceinline__ void store16(uint16_t* hi, uint16_t* lo, const float* v) {
-  uint16_t h[16], l[16];
+// 8 values as two pieces of rows of bfloat16 terms
+__device__ __forceinline__ void store8(uint16_t* hi, uint16_t* lo, const float* v) {
+  uint16_t h[8], l[8];
 #pragma unroll
-  for (int x = 0; x < 16; ++x) h[x] = hi_of(v[x]), l[x] = lo_of(v[x], h[x]);
-#pragma unroll
-  for (int y = 0; y < 2; ++y) {
-    uint4 a, b;
-    a.x = pair(h[8 * y], h[8 * y + 1]), a.y = pair(h[8 * y + 2], h[8 * y + 3]);
-    a.z = pair(h[8 * y + 4], h[8 * y + 5]), a.w = pair(h[8 * y + 6], h[8 * y + 7]);
-    b.x = pair(l[8 * y], l[8 * y + 1]), b.y = pair(l[8 * y + 2], l[8 * y + 3]);
-    b.z = pair(l[8 * y + 4], l[8 * y + 5]), b.w = pair(l[8 * y + 6], l[8 * y + 7]);
-    *reinterpret_cast<uint4*>(hi + 8 * y) = a;
-    *reinterpret_cast<uint4*>(lo + 8 * y) = b;
-  }
+  for (int x = 0; x < 8; ++x) h[x] = hi_of(v[x]), l[x] = lo_of(v[x], h[x]);
+  *reinterpret_cast<uint4*>(hi) = make_uint4(pair(h[0], h[1]), pair(h[2], h[3]), pair(h[4], h[5]), pair(h[6], h[7]));
+  *reinterpret_cast<uint4*>(lo) = make_uint4(pair(l[0], l[1]), pair(l[2], l[3]), pair(l[4], l[5]), pair(l[6], l[7]));
 }
 
 // four values of a row of P as two terms: P is [2][64][64] per (chunk, head)
@@ -93,22 +85,70 @@ struct ChunkBuffers {
 
 template <int DP>
 constexpr int prepare_words() {      // LDS of la_prepare in floats, without the chunk's products T [4][DP]
-  constexpr int a = 2 * kChunk * DP;                           // decays and q, or cosines and sines
+  constexpr int a = 2 * kChunk * DP;                           // decays and q
   constexpr int b = 4 * kChunk * (DP + kPad) / 2;              // q and k in two terms
-  constexpr int c = (2 * DP * kTS + 2 * kChunk * kTS) / 2;     // k transposed and v transposed in two terms
+  constexpr int c = (2 * DP * kTS + 2 * 128 * kTS) / 2;        // k transposed and 128 columns of v transposed, in two terms
   return a > b ? (a > c ? a : c) : (b > c ? b : c);
 }
 
+constexpr int kPrepThreads = 512;
+
+// P of the keys j = 4 m + kg, m = M0 and M1, of the wave's 16 tokens against the later ones of the same 16: 16 lanes share
+// the channels (pairs c = 2 r16 + 32 i), a key's product with the decays since runs along in registers.
+template <int DP, int M0, int M1>
+__device__ __forceinline__ void scores_within(const float* A, const float* Q, const float (*key)[DP / 32][2], int r16, int kg,
+                                              int row0, uint16_t* P) {
+  constexpr int CI = DP / 32;
+  float wk[2][CI][2], pd[2] = {0.f, 0.f};
+#pragma unroll
+  for (int y = 0; y < 2; ++y)
+#pragma unroll
+    for (int i = 0; i < CI; ++i) wk[y][i][0] = key[y][i][0], wk[y][i][1] = key[y][i][1];
+#pragma unroll
+  for (int i = 0; i < 16; ++i) {
+    float2 al[CI], q2[CI];
+#pragma unroll
+    for (int c = 0; c < CI; ++c) {
+      al[c] = *reinterpret_cast<const float2*>(A + (row0 + i) * DP + 2 * r16 + 32 * c);
+      q2[c] = *reinterpret_cast<const float2*>(Q + (row0 + i) * DP + 2 * r16 + 32 * c);
+    }
+#pragma unroll
+    for (int y = 0; y < 2; ++y) {
+      const int m = y ? M1 : M0;
+      if (4 * m > i) continue;
+      const bool past = 4 * m + 3 < i || 4 * m + kg < i;      // the key lies before token i: its product goes on
+      float dot = 0.f;
+#pragma unroll
+      for (int c = 0; c < CI; ++c) {
+        wk[y][c][0] *= past ? al[c].x : 1.0f;
+        wk[y][c][1] *= past ? al[c].y : 1.0f;
+        dot = fmaf(wk[y][c][0], q2[c].x, dot);
+        dot = fmaf(wk[y][c][1], q2[c].y, dot);
+      }
+      dot = row16_sum(dot);
+      if (r16 == i && 4 * m + kg <= i) pd[y] = dot;
+    }
+  }
+#pragma unroll
+  for (int y = 0; y < 2; ++y) {
+    const uint16_t hh = hi_of(pd[y]);
+    uint16_t* dst = P + (row0 + r16) * kChunk + row0 + 4 * (y ? M1 : M0) + kg;
+    dst[0] = hh;
+    dst[kPElems] = lo_of(pd[y], hh);
+  }
+}
+
 template <int DP, bool GATED>
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(kPrepThreads, DP <= 128 ? 4 : 2)
 la_prepare_kernel(LinearAttention a, const int32_t* __restrict__ chunks, ChunkBuffers buf, int vp) {
   extern __shared__ float lds[];
   constexpr int QS = DP + kPad;                  // row stride of q and k in LDS, in elements
-  constexpr int NP = (4 * DP + 255) / 256;       // (channel, 16 tokens) items a thread
-  constexpr int CT = DP / 16;
+  constexpr int NT = kPrepThreads;
+  constexpr int NP = (4 * DP + NT - 1) / NT;     // items of 16 values of q and k a thread
+  constexpr int CT = DP / 16, CI = DP / 32;
   float* T = lds + prepare_words<DP>();          // [4][DP]: the product of the decays of each 16 tokens
   const int h = blockIdx.x, ck = blockIdx.y, tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
-  const int r16 = lane & 15, kg = lane >> 4;
+  const int r16 = lane & 15, kg = lane >> 4, wq = w & 3, wh = w >> 2;
   const int tk = chunks[4 * ck + 1], n = chunks[4 * ck + 2];
   const size_t idx0 = (size_t)ck * a.heads + h;
   uint16_t* P = buf.p + idx0 * 2 * kPElems;
@@ -118,104 +158,97 @@ la_prepare_kernel(LinearAttention a, const int32_t* __restrict__ chunks, ChunkBu
   // P above the diagonal of the blocks of 32 tokens that la_finish takes whole
   if (w < 2) store_p4(P, 32 * w + r16, 32 * w + 16 + 4 * kg, zero4);
 
+  // A thread's items: gated, 16 tokens of one channel; fixed, 8 tokens of the two channels of a pair (those that are
+  // rotated together, or two neighbours behind the rotated ones).  Value x of an item: token tok(x), channel col(x).
+  const int half = a.rot >> 1;
+  auto c0_of = [&](int p) { const int item = tid + NT * p;
+                            if (GATED) return item % DP;
+                            const int i = item % (DP / 2);
+                            return i < half ? i : 2 * i; };
+  auto b_of = [&](int p) { const int item = tid + NT * p; return GATED ? item / DP : item / (DP / 2); };
+  auto live_item = [&](int p) { return b_of(p) < (GATED ? 4 : 8); };
+  auto col = [&](int p, int x) { return GATED || x < 8 ? c0_of(p) : c0_of(p) + (c0_of(p) < half ? half : 1); };
+  auto tok = [&](int p, int x) { return GATED ? 16 * b_of(p) + x : 8 * b_of(p) + (x & 7); };
+  float qv[NP][16], kv[NP][16];
+#pragma unroll
+  for (int p = 0; p < NP; ++p) {
+    if (!live_item(p)) continue;
+#pragma unroll
+    for (int x = 0; x < 16; ++x) {
+      const int t = tok(p, x), c = col(p, x);
+      const bool in = t < n && c < a.dim;
+      const float* row = proj + (size_t)t * a.ld + hd + c;
+      qv[p][x] = in ? row[a.off_q] : 0.f;
+      kv[p][x] = in ? row[a.off_k] : 0.f;
+    }
+  }
   float dec = 1.0f, l2 = 0.f;
-  float qv[NP][16], kv[NP][16], tail[NP];         // q and k of the thread's items
   if constexpr (GATED) {
     float* A = lds;                               // [64][DP] decays
     float* Q = lds + kChunk * DP;                 // [64][DP]
-    // decays: z = low w2^T + b, the wave's 16 tokens against all channels
-    {
-      const int j = 16 * w + r16, jc = j < n ? j : n - 1;
-      f32x4 acc[CT];
+    float key[2][CI][2];                          // the wave's keys of scores_within
 #pragma unroll
-      for (int ct = 0; ct < CT; ++ct) acc[ct] = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int y = 0; y < 2; ++y) {
+      const int j = 16 * wq + 4 * (y ? 3 - wh : wh) + kg;      // m = 0, 3 or 1, 2: equal work
+#pragma unroll
+      for (int i = 0; i < CI; ++i)
+#pragma unroll
+        for (int x = 0; x < 2; ++x) {
+          const int c = 2 * r16 + 32 * i + x;
+          key[y][i][x] = (j < n && c < a.dim) ? proj[(size_t)j * a.ld + a.off_k + hd + c] * a.k_scale : 0.f;
+        }
+    }
+    // decays: z = low w2^T + b, 16 tokens against half of the channels
+    {
+      const int j = 16 * wq + r16, jc = j < n ? j : n - 1;
+      f32x4 acc[CT / 2];
+#pragma unroll
+      for (int ct = 0; ct < CT / 2; ++ct) acc[ct] = f32x4{0.f, 0.f, 0.f, 0.f};
       for (int k0 = 0; k0 < a.rank; k0 += 4) {
         const int k = k0 + kg;
         const float lv = k < a.rank ? proj[(size_t)jc * a.ld + a.off_low + k] : 0.f;
 #pragma unroll
-        for (int ct = 0; ct < CT; ++ct) {
-          const int c = ct * 16 + r16;
+        for (int ct = 0; ct < CT / 2; ++ct) {
+          const int c = (wh * (CT / 2) + ct) * 16 + r16;
           const float wv = (k < a.rank && c < a.dim) ? a.w2[(size_t)(hd + c) * a.rank + k] : 0.f;
           acc[ct] = __builtin_amdgcn_mfma_f32_16x16x4f32(lv, wv, acc[ct], 0, 0, 0);
         }
       }
 #pragma unroll
-      for (int ct = 0; ct < CT; ++ct) {
-        const int c = ct * 16 + r16;
+      for (int ct = 0; ct < CT / 2; ++ct) {
+        const int c = (wh * (CT / 2) + ct) * 16 + r16;
         const float b = c < a.dim ? a.b2[hd + c] : 0.f;
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          const int t = 16 * w + 4 * kg + r;
+          const int t = 16 * wq + 4 * kg + r;
           A[t * DP + c] = (t < n && c < a.dim) ? gated_decay(acc[ct][r] + b, a.inv_tau) : 1.0f;
         }
       }
     }
-    for (int idx = tid; idx < kChunk * DP; idx += 256) {
-      const int t = idx / DP, c = idx % DP;
-      Q[idx] = (t < n && c < a.dim) ? proj[(size_t)t * a.ld + a.off_q + hd + c] * a.q_scale : 0.f;
-    }
-    __syncthreads();
-    // P inside the wave's 16 tokens: 16 lanes share the channels (pairs c = 2 r16 + 32 i), lane group kg holds the keys
-    // j = 4 m + kg with their running products
-    {
-      constexpr int CI = DP / 32;
-      float wk[4][CI][2], pd[4] = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-      for (int m = 0; m < 4; ++m) {
-        const int j = 16 * w + 4 * m + kg;
-#pragma unroll
-        for (int i = 0; i < CI; ++i)
-#pragma unroll
-          for (int x = 0; x < 2; ++x) {
-            const int c = 2 * r16 + 32 * i + x;
-            wk[m][i][x] = (j < n && c < a.dim) ? proj[(size_t)j * a.ld + a.off_k + hd + c] * a.k_scale : 0.f;
-          }
-      }
-#pragma unroll
-      for (int i = 0; i < 16; ++i) {
-        float2 al[CI], q2[CI];
-#pragma unroll
-        for (int c = 0; c < CI; ++c) {
-          al[c] = *reinterpret_cast<const float2*>(A + (16 * w + i) * DP + 2 * r16 + 32 * c);
-          q2[c] = *reinterpret_cast<const float2*>(Q + (16 * w + i) * DP + 2 * r16 + 32 * c);
-        }
-#pragma unroll
-        for (int m = 0; m < 4; ++m) {
-          if (4 * m > i) continue;
-          const bool past = 4 * m + 3 < i || 4 * m + kg < i;      // the key lies before token i: its product goes on
-          float dot = 0.f;
-#pragma unroll
-          for (int c = 0; c < CI; ++c) {
-            wk[m][c][0] *= past ? al[c].x : 1.0f;
-            wk[m][c][1] *= past ? al[c].y : 1.0f;
-            dot = fmaf(wk[m][c][0], q2[c].x, dot);
-            dot = fmaf(wk[m][c][1], q2[c].y, dot);
-          }
-          dot = row16_sum(dot);
-          if (r16 == i && 4 * m + kg <= i) pd[m] = dot;
-        }
-      }
-#pragma unroll
-      for (int m = 0; m < 4; ++m) {
-        const uint16_t hh = hi_of(pd[m]);
-        uint16_t* dst = P + (16 * w + r16) * kChunk + 16 * w + 4 * m + kg;
-        dst[0] = hh;
-        dst[kPElems] = lo_of(pd[m], hh);
-      }
-    }
-    // per (channel, 16 tokens): q decayed from the start of its 16, k decayed to the end of its own
 #pragma unroll
     for (int p = 0; p < NP; ++p) {
-      const int item = tid + 256 * p, c = item % DP, b = item / DP;
-      if (b >= 4) continue;
+      if (!live_item(p)) continue;
+#pragma unroll
+      for (int x = 0; x < 16; ++x) {
+        qv[p][x] *= a.q_scale;
+        kv[p][x] *= a.k_scale;
+        Q[tok(p, x) * DP + col(p, x)] = qv[p][x];
+      }
+    }
+    __syncthreads();
+    if (wh == 0) scores_within<DP, 0, 3>(A, Q, key, r16, kg, 16 * wq, P);
+    else scores_within<DP, 1, 2>(A, Q, key, r16, kg, 16 * wq, P);
+    // q decayed from the start of its 16, k decayed to the end of its own
+#pragma unroll
+    for (int p = 0; p < NP; ++p) {
+      if (!live_item(p)) continue;
+      const int c = c0_of(p), b = b_of(p);
       float al[16], run = 1.0f;
 #pragma unroll
       for (int x = 0; x < 16; ++x) {
-        const int t = 16 * b + x;
-        al[x] = A[t * DP + c];
+        al[x] = A[(16 * b + x) * DP + c];
         run *= al[x];
-        qv[p][x] = Q[t * DP + c] * run;
-        kv[p][x] = (t < n && c < a.dim) ? proj[(size_t)t * a.ld + a.off_k + hd + c] * a.k_scale : 0.f;
+        qv[p][x] *= run;
       }
       T[b * DP + c] = run;
       run = 1.0f;
@@ -225,70 +258,78 @@ la_prepare_kernel(LinearAttention a, const int32_t* __restrict__ chunks, ChunkBu
         run *= al[x];
       }
     }
+    __syncthreads();      // decays and q in LDS have been read; T is complete
   } else {
     dec = a.decay[h], l2 = log2f(dec);
-    const int half = a.rot >> 1;
-    float* cs = lds;                              // [64][half]
-    float* sn = lds + kChunk * (DP / 2);
-    for (int idx = tid; idx < n * half; idx += 256) {
-      const int t = idx / half, i = idx % half;
-      sincosf((float)a.positions[tk + t] * a.freq[i], &sn[t * half + i], &cs[t * half + i]);
-    }
-    __syncthreads();
 #pragma unroll
     for (int p = 0; p < NP; ++p) {
-      const int item = tid + 256 * p, c = item % DP, b = item / DP;
-      if (b >= 4) continue;
+      if (!live_item(p)) continue;
+      const int i = c0_of(p);
 #pragma unroll
-      for (int x = 0; x < 16; ++x) {
-        const int t = 16 * b + x;
-        const float* row = proj + (size_t)(t < n ? t : n - 1) * a.ld + hd;
-        const int tc = t < n ? t : n - 1;
-        qv[p][x] = (t < n && c < a.dim) ? rotated(row + a.off_q, c, a.rot, cs + tc * half, sn + tc * half) * a.q_scale : 0.f;
-        kv[p][x] = (t < n && c < a.dim) ? rotated(row + a.off_k, c, a.rot, cs + tc * half, sn + tc * half) * a.k_scale : 0.f;
+      for (int x = 0; x < 8; ++x) {
+        float cs = 1.0f, sn = 0.f;
+        if (i < half && tok(p, x) < n) {
+          const float* ang = a.angles + (size_t)(tk + tok(p, x)) * a.rot;
+          cs = ang[i], sn = ang[half + i];
+        }
+        const float q0 = qv[p][x], q1 = qv[p][x + 8], k0 = kv[p][x], k1 = kv[p][x + 8];
+        qv[p][x] = (q0 * cs - q1 * sn) * a.q_scale, qv[p][x + 8] = (q1 * cs + q0 * sn) * a.q_scale;
+        kv[p][x] = (k0 * cs - k1 * sn) * a.k_scale, kv[p][x + 8] = (k1 * cs + k0 * sn) * a.k_scale;
       }
     }
   }
-  __syncthreads();      // the first use of the workgroup's LDS is over; T is complete
 
   uint16_t* qh = (uint16_t*)lds;                  // [64][QS]
   uint16_t* ql = qh + kChunk * QS;
   uint16_t* kh = ql + kChunk * QS;
   uint16_t* kl = kh + kChunk * QS;
-  uint16_t* qg = buf.q + idx0 * 2 * kChunk * DP;
 #pragma unroll
   for (int p = 0; p < NP; ++p) {
-    const int item = tid + 256 * p, c = item % DP, b = item / DP;
-    if (b >= 4) continue;
-    float before = 1.0f;
-    tail[p] = 1.0f;
+    if (!live_item(p)) continue;
+#pragma unroll
+    for (int x = 0; x < 16; ++x) {
+      const int at = tok(p, x) * QS + col(p, x);
+      const uint16_t q0 = hi_of(qv[p][x]), k0 = hi_of(kv[p][x]);
+      qh[at] = q0, ql[at] = lo_of(qv[p][x], q0);
+      kh[at] = k0, kl[at] = lo_of(kv[p][x], k0);
+    }
+    // k decayed on to the chunk's end
     if constexpr (GATED) {
+      const int c = c0_of(p), b = b_of(p);
+      float f = 1.0f, whole = 1.0f;
 #pragma unroll
       for (int y = 0; y < 4; ++y) {
         const float t = T[y * DP + c];
-        before *= y < b ? t : 1.0f;
-        tail[p] *= y > b ? t : 1.0f;
+        f *= y > b ? t : 1.0f;
+        whole *= t;
       }
-      if (b == 3) buf.d[idx0 * DP + c] = before * T[3 * DP + c];
-    } else {
-      if (b == 3) buf.d[idx0 * DP + c] = pow_int(l2, n);
-    }
+      if (b == 3) buf.d[idx0 * DP + c] = whole;
 #pragma unroll
-    for (int x = 0; x < 16; ++x) {
-      const int t = 16 * b + x;
-      const uint16_t q0 = hi_of(qv[p][x]), k0 = hi_of(kv[p][x]);
-      qh[t * QS + c] = q0, ql[t * QS + c] = lo_of(qv[p][x], q0);
-      kh[t * QS + c] = k0, kl[t * QS + c] = lo_of(kv[p][x], k0);
-      const float qb = qv[p][x] * (GATED ? before : pow_int(l2, t + 1));
-      const uint16_t g = hi_of(qb);
-      qg[t * DP + c] = g;
-      qg[kChunk * DP + t * DP + c] = lo_of(qb, g);
+      for (int x = 0; x < 16; ++x) kv[p][x] *= f;
+    } else {
+#pragma unroll
+      for (int x = 0; x < 8; ++x) {
+        const float f = tok(p, x) < n ? pow_int(l2, n - 1 - tok(p, x)) : 0.f;
+        kv[p][x] *= f, kv[p][x + 8] *= f;
+      }
+      if (b_of(p) == 0) buf.d[idx0 * DP + col(p, 0)] = buf.d[idx0 * DP + col(p, 8)] = pow_int(l2, n);
     }
   }
+  // v of the first columns is on its way while the scores are made
+  float vv[16];
+  auto ask_v = [&](int v0) {
+    const int v = v0 + (tid & 127);
+#pragma unroll
+    for (int x = 0; x < 16; ++x) {
+      const int t = 16 * (tid >> 7) + x;
+      vv[x] = (t < n && v < a.vdim) ? proj[(size_t)t * a.ld + a.off_v + h * a.vdim + v] : 0.f;
+    }
+  };
+  ask_v(0);
   __syncthreads();
 
   // P between different 16s (gated), or all of P on and below the diagonal (fixed): D[j][i] with A = k, B = q
-  for (int job = w; job < (GATED ? 6 : 10); job += 4) {
+  for (int job = w; job < (GATED ? 6 : 10); job += 8) {
     int I, J;
     if constexpr (GATED) {
       I = job == 0 ? 3 : job == 1 ? 2 : job == 2 ? 3 : job == 3 ? 1 : job == 4 ? 2 : 3;
@@ -316,39 +357,52 @@ la_prepare_kernel(LinearAttention a, const int32_t* __restrict__ chunks, ChunkBu
     for (int r = 0; r < 4; ++r) pv[r] = GATED ? acc[r] : (j0 + r <= i ? acc[r] * pow_int(l2, i - j0 - r) : 0.f);
     store_p4(P, i, j0, pv);
   }
+  // B q for la_finish, 8 channels at a time: what is in LDS, decayed from the chunk's start
+  uint16_t* qg = buf.q + idx0 * 2 * kChunk * DP;
+  for (int idx = tid; idx < kChunk * DP / 8; idx += NT) {
+    const int t = idx / (DP / 8), c = idx % (DP / 8) * 8;
+    bf16x8 fh = frag(qh + t * QS + c), fl = frag(ql + t * QS + c);
+    if (!GATED || t >= 16) {
+      float f[8];
+      if constexpr (GATED) {
+#pragma unroll
+        for (int x = 0; x < 8; ++x)
+          f[x] = T[c + x] * (t >= 32 ? T[DP + c + x] : 1.0f) * (t >= 48 ? T[2 * DP + c + x] : 1.0f);
+      } else {
+        const float g = pow_int(l2, t + 1);
+#pragma unroll
+        for (int x = 0; x < 8; ++x) f[x] = g;
+      }
+      scale_frag(fh, fl, f);
+    }
+    *reinterpret_cast<bf16x8*>(qg + t * DP + c) = fh;
+    *reinterpret_cast<bf16x8*>(qg + kChunk * DP + t * DP + c) = fl;
+  }
   __syncthreads();      // q and k in LDS have been read
 
-  // U: k decayed to the chunk's end, transposed, against v, 64 columns of it at a time
+  // U: k decayed to the chunk's end, transposed, against v, 128 columns of it at a time
   uint16_t* kth = (uint16_t*)lds;                 // [DP][kTS]
   uint16_t* ktl = kth + DP * kTS;
-  uint16_t* vth = ktl + DP * kTS;                 // [64][kTS]
-  uint16_t* vtl = vth + kChunk * kTS;
+  uint16_t* vth = ktl + DP * kTS;                 // [128][kTS]
+  uint16_t* vtl = vth + 128 * kTS;
 #pragma unroll
   for (int p = 0; p < NP; ++p) {
-    const int item = tid + 256 * p, c = item % DP, b = item / DP;
-    if (b >= 4) continue;
-    float kt[16];
-#pragma unroll
-    for (int x = 0; x < 16; ++x) {
-      const int t = 16 * b + x;
-      kt[x] = kv[p][x] * (GATED ? tail[p] : (t < n ? pow_int(l2, n - 1 - t) : 0.f));
-    }
-    store16(kth + c * kTS + 16 * b, ktl + c * kTS + 16 * b, kt);
+    if (!live_item(p)) continue;
+    const int t = tok(p, 0);
+    store8(kth + col(p, 0) * kTS + t, ktl + col(p, 0) * kTS + t, kv[p]);
+    if constexpr (GATED) store8(kth + col(p, 0) * kTS + t + 8, ktl + col(p, 0) * kTS + t + 8, kv[p] + 8);
+    else store8(kth + col(p, 8) * kTS + t, ktl + col(p, 8) * kTS + t, kv[p] + 8);
   }
   float* U = buf.u + idx0 * (size_t)vp * DP;
-  for (int v0 = 0; v0 < vp; v0 += 64) {
+  for (int v0 = 0; v0 < vp; v0 += 128) {
     if (v0) __syncthreads();
     {
-      const int v = v0 + lane;
-      float vv[16];
-#pragma unroll
-      for (int x = 0; x < 16; ++x) {
-        const int t = 16 * w + x;
-        vv[x] = (t < n && v < a.vdim) ? proj[(size_t)t * a.ld + a.off_v + h * a.vdim + v] : 0.f;
-      }
-      store16(vth + lane * kTS + 16 * w, vtl + lane * kTS + 16 * w, vv);
+      const int at = (tid & 127) * kTS + 16 * (tid >> 7);
+      store8(vth + at, vtl + at, vv);
+      store8(vth + at + 8, vtl + at + 8, vv + 8);
     }
     __syncthreads();
+    if (v0 + 128 < vp) ask_v(v0 + 128);
     const int vt = v0 + 16 * w;
     if (vt < vp) {
       bf16x8 bh[2], bl[2];
@@ -467,23 +521,31 @@ la_finish_kernel(LinearAttention a, const int32_t* __restrict__ chunks, ChunkBuf
         vl[x][s][y8] = (__bf16)(f - (float)hb);
       }
   }
+  // the state's first fragments are on their way before the tiles above have arrived
+  bf16x8 sh[2][VT], sl[2][VT];
+  auto ask_s = [&](int ks) {
+#pragma unroll
+    for (int x = 0; x < VT; ++x) {
+      const int v0 = (w + 4 * x) * 16;
+      const uint16_t* p = S + (size_t)((v0 < vp ? v0 : 0) + r16) * DP + ks * 32 + kg * 8;
+      sh[ks & 1][x] = frag(p), sl[ks & 1][x] = frag(p + (size_t)vp * DP);
+    }
+  };
+  ask_s(0);
   __syncthreads();
   // D[v][i]: S0^T (B q), then v^T P^T
 #pragma unroll
   for (int ks = 0; ks < DP / 32; ++ks) {
     const int at = ks * 32 + kg * 8;
+    if (ks + 1 < DP / 32) ask_s(ks + 1);
     bf16x8 bh[4], bl[4];
 #pragma unroll
     for (int it = 0; it < 4; ++it)
       bh[it] = frag(qh + (it * 16 + r16) * QS + at), bl[it] = frag(ql + (it * 16 + r16) * QS + at);
 #pragma unroll
-    for (int x = 0; x < VT; ++x) {
-      const int v = (w + 4 * x) * 16 + r16;
-      if ((w + 4 * x) * 16 >= vp) continue;
-      const bf16x8 ah = frag(S + (size_t)v * DP + at), al = frag(S + (size_t)vp * DP + (size_t)v * DP + at);
+    for (int x = 0; x < VT; ++x)      // (columns beyond vdim are computed from others' state and never stored)
 #pragma unroll
-      for (int it = 0; it < 4; ++it) acc[x][it] = mfma3(ah, al, bh[it], bl[it], acc[x][it]);
-    }
+      for (int it = 0; it < 4; ++it) acc[x][it] = mfma3(sh[ks & 1][x], sl[ks & 1][x], bh[it], bl[it], acc[x][it]);
   }
 #pragma unroll
   for (int s = 0; s < 2; ++s)
@@ -500,7 +562,7 @@ la_finish_kernel(LinearAttention a, const int32_t* __restrict__ chunks, ChunkBuf
 #pragma unroll
     for (int x = 0; x < VT; ++x)
 #pragma unroll
-      for (int r = 0; r < 4; ++r) ss = fmaf(acc[x][it][r], acc[x][it][r], ss);
+      for (int r = 0; r < 4; ++r) ss = (w + 4 * x) * 16 < vp ? fmaf(acc[x][it][r], acc[x][it][r], ss) : ss;
     ss += __shfl_xor(ss, 16, 64);
     ss += __shfl_xor(ss, 32, 64);
     if (kg == 0) sums[w][it * 16 + r16] = ss;
@@ -550,7 +612,8 @@ static void launch_prepare(const LinearAttention& a, const int32_t* chunks, cons
                            hipStream_t stream) {
   const size_t lds = (size_t)(prepare_words<DP>() + 4 * DP) * sizeof(float);
   (void)hipFuncSetAttribute((const void*)la_prepare_kernel<DP, GATED>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
-  hipLaunchKernelGGL((la_prepare_kernel<DP, GATED>), dim3(a.heads, n_chunks), dim3(256), lds, stream, a, chunks, buf, vp);
+  hipLaunchKernelGGL((la_prepare_kernel<DP, GATED>), dim3(a.heads, n_chunks), dim3(kPrepThreads), lds, stream, a, chunks, buf,
+                     vp);
 }
 
 // The columns of S as these kernels pad them, and the most they take.
@@ -563,16 +626,16 @@ extern "C" int atoma_linear_attention_padded_vdim(int vdim) { return (vdim + 15)
 // atoma_linear_attention_scan.
 extern "C" int atoma_linear_attention_chunked(const float* proj, const int32_t* at, const float* decay, const float* w2,
                                               const float* b2, float inv_tau, const int32_t* positions, const float* freq,
-                                              int rot, float q_scale, float k_scale, const float* norm_w, float eps,
+                                              const float* angles, int rot, float q_scale, float k_scale, const float* norm_w, float eps,
                                               const int32_t* q_start, const int32_t* state_slots, float* state,
                                               int heads, int dim, int vdim, void* y, const int32_t* chunks,
                                               int n_chunks, const int32_t* entries, int n_long, void* wp, void* wq,
                                               float* wd, float* wu, void* ws, hipStream_t stream) {
   if (n_chunks <= 0 || n_long <= 0) return 0;
-  const LinearAttention a = linear_attention_args(proj, at, decay, w2, b2, inv_tau, positions, freq, rot, q_scale, k_scale,
-                                                  norm_w, eps, q_start, state_slots, state, heads, dim, vdim);
+  const LinearAttention a = linear_attention_args(proj, at, decay, w2, b2, inv_tau, positions, freq, angles, rot, q_scale,
+                                                  k_scale, norm_w, eps, q_start, state_slots, state, heads, dim, vdim);
   constexpr int DP = ATOMA_LA_DP;
-  if (!linear_attention_ok(a) || (dim + 31) / 32 * 32 != DP || vdim > 512 || n_chunks > 65535 || n_long > 65535)
+  if (!linear_attention_ok(a) || (rot > 0 && angles == nullptr) || (dim + 31) / 32 * 32 != DP || vdim > 512 || n_chunks > 65535 || n_long > 65535)
     return ATOMA_ERR_SHAPE;
   const ChunkBuffers buf{(uint16_t*)wp, (uint16_t*)wq, wd, wu, (uint16_t*)ws};
   const int vp = atoma_linear_attention_padded_vdim(vdim);

@@ -1242,12 +1242,26 @@ def linear_attention_plan(counts, chunked_from: int):
     return np.asarray(rows + entries, dtype=np.int32).reshape(-1), (len(rows), len(entries), short)
 
 
+def linear_attention_angles(positions: torch.Tensor, freq: torch.Tensor) -> torch.Tensor:
+    """[T, 2 n] float32: the cosines, then the sines of positions[t] * freq[i] (n frequencies), angles in float32."""
+    _dev(positions, freq)
+    t = positions.numel()
+    _i32(positions, "positions", t)
+    _f32(freq, "frequencies")
+    out = torch.empty((t, 2 * freq.numel()), dtype=torch.float32, device=freq.device)
+    _check(_module("linear_attention").atoma_linear_attention_angles(_p(positions), _p(freq), freq.numel(), _p(out), t,
+                                                                     _stream()), "linear_attention_angles")
+    return out
+
+
 def linear_attention(proj: torch.Tensor, sizes: LinearAttentionSizes, w: LinearAttentionTensors, positions, q_start,
-                     state_slots, state: torch.Tensor, out_dtype: torch.dtype, plan, chunked_from: int) -> torch.Tensor:
+                     state_slots, state: torch.Tensor, out_dtype: torch.dtype, plan, chunked_from: int,
+                     angles: Optional[torch.Tensor] = None) -> torch.Tensor:
     """y [T, heads vdim] in ``out_dtype`` from ``proj`` float32 [T, ld]: the recurrence over every entry's tokens from and
     into the requests' rows of ``state`` float32 [slots, heads vdim dim], its result normed head by head and gated.
     ``plan``: (int32 device tensor, meta) of ``linear_attention_plan`` for the same ``chunked_from``, None only if that is
-    0; entries cut into chunks need ``out_dtype`` bfloat16."""
+    0; entries cut into chunks need ``out_dtype`` bfloat16.  ``angles``: what ``linear_attention_angles`` makes of the
+    positions, which chunks with rotated columns read; made here where they are needed and not given."""
     _dev(proj, positions, q_start, state_slots, state, w.decay, w.w2, w.b2, w.freq, w.norm)
     t, n_entries = proj.shape[0], state_slots.numel()
     h, dim, vdim = sizes.heads, sizes.dim, sizes.vdim
@@ -1278,11 +1292,11 @@ def linear_attention(proj: torch.Tensor, sizes: LinearAttentionSizes, w: LinearA
     low = sizes.low or (0, 0)
     ld = proj.stride(0) if t > 1 else proj.shape[1]
     at = (ctypes.c_int32 * 7)(ld, *(int(o) for o in sizes.offsets), int(low[0]), int(low[1]))
-    args = (_p(proj), at, _p(w.decay), _p(w.w2), _p(w.b2), ctypes.c_float(sizes.inv_tau), _p(positions), _p(w.freq),
-            int(sizes.rot), ctypes.c_float(sizes.q_scale), ctypes.c_float(sizes.k_scale), _p(w.norm),
+    first = (_p(proj), at, _p(w.decay), _p(w.w2), _p(w.b2), ctypes.c_float(sizes.inv_tau), _p(positions), _p(w.freq))
+    rest = (int(sizes.rot), ctypes.c_float(sizes.q_scale), ctypes.c_float(sizes.k_scale), _p(w.norm),
             ctypes.c_float(sizes.eps), _p(q_start), _p(state_slots), _p(state), h, dim, vdim)
     n_chunks, n_long, short = (0, 0, None)
-    if chunked_from:
+    if plan is not None:
         arr, (n_chunks, n_long, short) = plan
         _i32(arr, "chunks", 4 * (n_chunks + n_long))
     if short != 0:
@@ -1291,12 +1305,16 @@ def linear_attention(proj: torch.Tensor, sizes: LinearAttentionSizes, w: LinearA
         tb = 16 if short is None else next(b for b in (1, 2, 4, 8, 16) if b >= min(short, 16))
         o = torch.empty((t, h * vdim), dtype=torch.float32, device=proj.device) \
             if lib.atoma_linear_attention_needs_o(dim, vdim) else None
-        _check(lib.atoma_linear_attention_scan(*args, _p(y), _code(y, "y"), _p(o), n_entries, tb,
+        _check(lib.atoma_linear_attention_scan(*first, *rest, _p(y), _code(y, "y"), _p(o), n_entries, tb,
                                                int(chunked_from), _stream()), "linear_attention_scan")
     if n_chunks:
         _need(out_dtype is torch.bfloat16 and vdim <= LINEAR_ATTENTION_CHUNKED_MAX_VDIM,
               "linear_attention: chunks leave bfloat16, and up to 512 value columns a head")
         dp, vp = -(-dim // 32) * 32, -(-vdim // 16) * 16
+        if sizes.rot:
+            if angles is None:
+                angles = linear_attention_angles(positions, w.freq)
+            _f32(angles, "angles", t * sizes.rot)
         lib = load_hip_module(*linear_attention_module(dp))
         n = n_chunks * h
         bf = dict(dtype=torch.bfloat16, device=proj.device)
@@ -1305,7 +1323,7 @@ def linear_attention(proj: torch.Tensor, sizes: LinearAttentionSizes, w: LinearA
         wp, wq = torch.empty((n, 2, c, c), **bf), torch.empty((n, 2, c, dp), **bf)
         wd, wu, ws = torch.empty((n, dp), **f32), torch.empty((n, vp, dp), **f32), torch.empty((n, 2, vp, dp), **bf)
         _check(lib.atoma_linear_attention_chunked(
-            *args, _p(y), _p(arr), n_chunks, ctypes.c_void_p(arr.data_ptr() + 16 * n_chunks), n_long, _p(wp), _p(wq),
+            *first, _p(angles), *rest, _p(y), _p(arr), n_chunks, ctypes.c_void_p(arr.data_ptr() + 16 * n_chunks), n_long, _p(wp), _p(wq),
             _p(wd), _p(wu), _p(ws), _stream()), "linear_attention_chunked")
     return y
 

@@ -483,21 +483,27 @@ class DecayedLinearAttention(Mixer):
         return ("linear_attention_chunks", self.chunked)
 
     def step_planner(self, page_size: int, cache_dtype: torch.dtype):
-        """(key, fn(starts, counts, bucket_tokens) -> (int32 array, meta)): the chunks of long entries."""
-        if not self.chunked:
-            return None
+        """(key, fn(starts, counts, bucket_tokens) -> (int32 array, meta)): the chunks of long entries, and how long the
+        others are."""
         chunked = self.chunked
         return self._plan_key(), lambda starts, counts, bucket: ops.linear_attention_plan(counts, chunked)
 
     def forward(self, x, ctx, cache):
         proj = linear(x, self.w_in, torch.float32, tiled=self.w_in_tiled)
         plan = getattr(ctx, "plans", {}).get(self._plan_key())
-        if plan is None and self.chunked:
+        if plan is None:
             # a caller without a step planner (a test of the part alone): plan here and now
             arr, meta = ops.linear_attention_plan(ctx.h_counts, self.chunked)
             plan = (torch.from_numpy(arr).to(x.device), meta)
+        angles = None
+        if self.rot and plan[1][0]:
+            # the rotation's cosines and sines for chunks: made once a step for all layers that turn alike
+            key = ("linear_attention_angles", self.rotary_base, self.rot)
+            angles = ctx.scratch.get(key)
+            if angles is None:
+                angles = ctx.scratch[key] = ops.linear_attention_angles(ctx.positions, self.tensors.freq)
         y = ops.linear_attention(proj, self.sizes, self.tensors, ctx.positions, ctx.q_start, ctx.state_slots, cache.state,
-                                 x.dtype, plan, self.chunked)
+                                 x.dtype, plan, self.chunked, angles)
         return linear_delta(y, self.w_o, None, self.w_o_tiled)
 
 
