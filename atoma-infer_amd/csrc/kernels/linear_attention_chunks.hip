@@ -85,7 +85,7 @@ struct ChunkBuffers {
 
 template <int DP>
 constexpr int prepare_words() {      // LDS of la_prepare in floats, without the chunk's products T [4][DP]
-  constexpr int a = 2 * kChunk * DP;                           // decays and q
+  constexpr int a = 2 * kChunk * (DP + 4);                     // decays and q
   constexpr int b = 4 * kChunk * (DP + kPad) / 2;              // q and k in two terms
   constexpr int c = (2 * DP * kTS + 2 * 128 * kTS) / 2;        // k transposed and 128 columns of v transposed, in two terms
   return a > b ? (a > c ? a : c) : (b > c ? b : c);
@@ -109,8 +109,8 @@ __device__ __forceinline__ void scores_within(const float* A, const float* Q, co
     float2 al[CI], q2[CI];
 #pragma unroll
     for (int c = 0; c < CI; ++c) {
-      al[c] = *reinterpret_cast<const float2*>(A + (row0 + i) * DP + 2 * r16 + 32 * c);
-      q2[c] = *reinterpret_cast<const float2*>(Q + (row0 + i) * DP + 2 * r16 + 32 * c);
+      al[c] = *reinterpret_cast<const float2*>(A + (row0 + i) * (DP + 4) + 2 * r16 + 32 * c);
+      q2[c] = *reinterpret_cast<const float2*>(Q + (row0 + i) * (DP + 4) + 2 * r16 + 32 * c);
     }
 #pragma unroll
     for (int y = 0; y < 2; ++y) {
@@ -184,8 +184,9 @@ la_prepare_kernel(LinearAttention a, const int32_t* __restrict__ chunks, ChunkBu
   }
   float dec = 1.0f, l2 = 0.f;
   if constexpr (GATED) {
-    float* A = lds;                               // [64][DP] decays
-    float* Q = lds + kChunk * DP;                 // [64][DP]
+    constexpr int AS = DP + 4;                    // (rows four apart fall into different banks)
+    float* A = lds;                               // [64][AS] decays
+    float* Q = lds + kChunk * AS;                 // [64][AS]
     float key[2][CI][2];                          // the wave's keys of scores_within
 #pragma unroll
     for (int y = 0; y < 2; ++y) {
@@ -204,15 +205,23 @@ la_prepare_kernel(LinearAttention a, const int32_t* __restrict__ chunks, ChunkBu
       f32x4 acc[CT / 2];
 #pragma unroll
       for (int ct = 0; ct < CT / 2; ++ct) acc[ct] = f32x4{0.f, 0.f, 0.f, 0.f};
-      for (int k0 = 0; k0 < a.rank; k0 += 4) {
-        const int k = k0 + kg;
-        const float lv = k < a.rank ? proj[(size_t)jc * a.ld + a.off_low + k] : 0.f;
+      constexpr int KU = CT <= 8 ? 2 : 1;      // steps of 4 low-rank values whose operands are asked for together
+      for (int k0 = 0; k0 < a.rank; k0 += 4 * KU) {
+        float lv[KU], wv[KU][CT / 2];
 #pragma unroll
-        for (int ct = 0; ct < CT / 2; ++ct) {
-          const int c = (wh * (CT / 2) + ct) * 16 + r16;
-          const float wv = (k < a.rank && c < a.dim) ? a.w2[(size_t)(hd + c) * a.rank + k] : 0.f;
-          acc[ct] = __builtin_amdgcn_mfma_f32_16x16x4f32(lv, wv, acc[ct], 0, 0, 0);
+        for (int u = 0; u < KU; ++u) {
+          const int k = k0 + 4 * u + kg;
+          lv[u] = k < a.rank ? proj[(size_t)jc * a.ld + a.off_low + k] : 0.f;
+#pragma unroll
+          for (int ct = 0; ct < CT / 2; ++ct) {
+            const int c = (wh * (CT / 2) + ct) * 16 + r16;
+            wv[u][ct] = (k < a.rank && c < a.dim) ? a.w2[(hd + c) * a.rank + k] : 0.f;
+          }
         }
+#pragma unroll
+        for (int u = 0; u < KU; ++u)
+#pragma unroll
+          for (int ct = 0; ct < CT / 2; ++ct) acc[ct] = __builtin_amdgcn_mfma_f32_16x16x4f32(lv[u], wv[u][ct], acc[ct], 0, 0, 0);
       }
 #pragma unroll
       for (int ct = 0; ct < CT / 2; ++ct) {
@@ -221,7 +230,7 @@ la_prepare_kernel(LinearAttention a, const int32_t* __restrict__ chunks, ChunkBu
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           const int t = 16 * wq + 4 * kg + r;
-          A[t * DP + c] = (t < n && c < a.dim) ? gated_decay(acc[ct][r] + b, a.inv_tau) : 1.0f;
+          A[t * AS + c] = (t < n && c < a.dim) ? gated_decay(acc[ct][r] + b, a.inv_tau) : 1.0f;
         }
       }
     }
@@ -232,7 +241,7 @@ la_prepare_kernel(LinearAttention a, const int32_t* __restrict__ chunks, ChunkBu
       for (int x = 0; x < 16; ++x) {
         qv[p][x] *= a.q_scale;
         kv[p][x] *= a.k_scale;
-        Q[tok(p, x) * DP + col(p, x)] = qv[p][x];
+        Q[tok(p, x) * AS + col(p, x)] = qv[p][x];
       }
     }
     __syncthreads();
@@ -246,7 +255,7 @@ la_prepare_kernel(LinearAttention a, const int32_t* __restrict__ chunks, ChunkBu
       float al[16], run = 1.0f;
 #pragma unroll
       for (int x = 0; x < 16; ++x) {
-        al[x] = A[(16 * b + x) * DP + c];
+        al[x] = A[(16 * b + x) * AS + c];
         run *= al[x];
         qv[p][x] *= run;
       }
