@@ -1,8 +1,8 @@
 """The cache manager: which pages and which state slot each request holds.
 
 A thin face of the native manager (csrc/host/cache_manager.cpp).  It knows nothing of tensors: groups are
-(page size, number of pages, window) triples, requests are integers.  ``CachePool`` (pool.py) owns the device
-memory that the page numbers index.
+(page size, number of pages, window and what it keeps beside) records, requests are integers.  ``CachePool`` (pool.py)
+owns the device memory that the page numbers index.
 """
 from __future__ import annotations
 
@@ -30,6 +30,8 @@ class GroupGeometry:
     window: Optional[int] = None
     #: chunks of this many positions instead of a window: a token sees the keys of its own chunk only
     chunk: Optional[int] = None
+    #: with a window: a request's first tokens, which stay beside it
+    keep_first: int = 0
 
 
 _lib = None
@@ -40,7 +42,8 @@ def _host():
     if _lib is None:
         lib = load_host_library()
         lib.cm_create.restype = ctypes.c_void_p
-        lib.cm_create.argtypes = [ctypes.c_int, ctypes.c_void_p, ctypes.c_void_p, ctypes.c_void_p, ctypes.c_int]
+        lib.cm_create.argtypes = [ctypes.c_int, ctypes.c_void_p, ctypes.c_void_p, ctypes.c_void_p, ctypes.c_void_p,
+                                  ctypes.c_int]
         lib.cm_destroy.argtypes = [ctypes.c_void_p]
         lib.cm_destroy.restype = None
         for name in ("cm_add_request", "cm_free", "cm_state_slot"):
@@ -86,7 +89,8 @@ class CacheManager:
         if any(g.window and g.chunk for g in groups):
             raise CacheError("a group keeps a window or chunks, not both")
         win = _i32((-g.chunk if g.chunk else (g.window or 0)) for g in groups)      # chunks travel as negative windows
-        self._h = lib.cm_create(len(self.groups), ps.ctypes.data, npg.ctypes.data, win.ctypes.data,
+        keep = _i32(g.keep_first for g in groups)
+        self._h = lib.cm_create(len(self.groups), ps.ctypes.data, npg.ctypes.data, win.ctypes.data, keep.ctypes.data,
                                 self.num_state_slots)
         if not self._h:
             raise CacheError(f"invalid cache geometry: {self.groups}, {num_state_slots} state slots")

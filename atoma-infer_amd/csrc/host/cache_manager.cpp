@@ -1,9 +1,9 @@
 // Page tables and free lists of the paged cache, and the slots of per-request fixed-size state.
 //
 // Layers with equal cache needs form a group; each group has its own pool of pages (its own page numbers) and each
-// request has one block table per group.  A group may keep all tokens or only a window of the last W: pages
-// that a window has passed are given back while the request is still running.  Pages come from a LIFO free
-// list, so the page freed last is used next (the reference's allocator pops from a Vec the same way:
+// request has one block table per group.  A group may keep all tokens or only a window of the last W (and, where it is
+// asked to, the first K beside them): pages that a window has passed are given back while the request is still
+// running.  Pages come from a LIFO free list, so the page freed last is used next (the reference's allocator pops from a Vec the same way:
 // backends/vllm/src/block_allocator.rs:59-111).  Unlike the reference (backends/vllm/src/block_manager.rs:195-237,
 // 294-377) pages are reserved for whatever length the next step reaches, any number at a time, and all groups
 // together or not at all.
@@ -24,6 +24,8 @@ struct Group {
   // (chunks count from the request's first position), so everything before the chunk of the next token is dead.
   // Either way a request never needs more than the pages of `window` tokens and the page that the next token opens.
   bool chunked = false;
+  // with a window: the tokens from a request's first on that the window never loses; their pages stay
+  int keep = 0;
   std::vector<int32_t> free_list;
   std::vector<uint8_t> in_use;
 };
@@ -32,7 +34,7 @@ struct Request {
   int state_slot = -1;
   int64_t reserved_len = 0;                   // pages cover positions [0, reserved_len) except released ones
   std::vector<std::vector<int32_t>> tables;   // per group; -1 marks a released entry
-  std::vector<int64_t> first_live;            // per group: index of the first entry not released
+  std::vector<int64_t> first_live;            // per group: entries that the window has passed (all released but the kept ones)
 };
 
 struct Manager {
@@ -55,8 +57,17 @@ int64_t pages_needed(const Manager& m, const Request* r, size_t gi, int64_t new_
   return want > have ? want - have : 0;
 }
 
+// pages at a request's beginning that its window never releases
+inline int64_t kept_blocks(const Group& g) { return g.window > 0 ? ceil_div(g.keep, g.page_size) : 0; }
+
+// pages that a request needs once its window has moved on: the window, the page that the next token opens, the kept ones
+inline int64_t steady_blocks(const Group& g) { return blocks_for(g, g.window) + 1 + kept_blocks(g); }
+
 // pages of request r in group gi that are still held (table entries that a window has not released)
-int64_t live_pages(const Request& r, size_t gi) { return (int64_t)r.tables[gi].size() - r.first_live[gi]; }
+int64_t live_pages(const Manager& m, const Request& r, size_t gi) {
+  const int64_t kept = kept_blocks(m.groups[gi]);
+  return (int64_t)r.tables[gi].size() - r.first_live[gi] + (kept < r.first_live[gi] ? kept : r.first_live[gi]);
+}
 
 }  // namespace
 
@@ -65,11 +76,13 @@ extern "C" {
 enum { CM_OK = 0, CM_NO_PAGES = -1, CM_EXISTS = -2, CM_UNKNOWN = -3, CM_NO_SLOT = -4, CM_BAD_ARG = -5,
        CM_CORRUPT = -6 };
 
+// windows[i]: 0 keeps everything, w > 0 a window of w, -c < 0 chunks of c; keeps[i]: the first tokens of a request that a
+// window keeps beside (0 without a window)
 void* cm_create(int n_groups, const int32_t* page_sizes, const int32_t* num_pages, const int32_t* windows,
-                int n_state_slots) {
+                const int32_t* keeps, int n_state_slots) {
   if (n_groups < 0 || n_state_slots < 0) return nullptr;
   for (int i = 0; i < n_groups; ++i)
-    if (page_sizes[i] <= 0 || num_pages[i] < 0) return nullptr;
+    if (page_sizes[i] <= 0 || num_pages[i] < 0 || keeps[i] < 0 || (keeps[i] > 0 && windows[i] <= 0)) return nullptr;
   Manager* m = new Manager();
   m->groups.resize(n_groups);
   for (int i = 0; i < n_groups; ++i) {
@@ -78,6 +91,7 @@ void* cm_create(int n_groups, const int32_t* page_sizes, const int32_t* num_page
     g.num_pages = num_pages[i];
     g.window = windows[i] < 0 ? -windows[i] : windows[i];      // (a negative entry: chunks of that many positions)
     g.chunked = windows[i] < 0;
+    g.keep = keeps[i];
     g.in_use.assign(g.num_pages, 0);
     g.free_list.reserve(g.num_pages);
     // page 0 is handed out first
@@ -117,12 +131,12 @@ int cm_can_reserve(void* h, int64_t id, int64_t new_len) {
 }
 
 // 1 if a request of new_len tokens could ever be held, with every page free.  A group with a window gives pages
-// back as the request moves on: it must hold the window and the page that the next token opens.
+// back as the request moves on: it must hold the window, the page that the next token opens and the pages it keeps.
 int cm_fits_at_all(void* h, int64_t new_len) {
   Manager* m = static_cast<Manager*>(h);
   for (const Group& g : m->groups) {
     int64_t need = blocks_for(g, new_len);
-    if (g.window > 0 && blocks_for(g, g.window) + 1 < need) need = blocks_for(g, g.window) + 1;
+    if (g.window > 0 && steady_blocks(g) < need) need = steady_blocks(g);
     if (need > g.num_pages) return 0;
   }
   return 1;
@@ -139,11 +153,11 @@ int cm_can_admit(void* h, int64_t total_len, int64_t first_len) {
     const Group& g = m->groups[gi];
     int64_t need = blocks_for(g, first_len);
     if (g.window > 0) {
-      const int64_t steady = blocks_for(g, g.window) + 1;
+      const int64_t steady = steady_blocks(g);
       const int64_t own = blocks_for(g, total_len) < steady ? blocks_for(g, total_len) : steady;
       if (own > need) need = own;
       for (const auto& kv : m->requests) {
-        const int64_t lack = steady - live_pages(kv.second, gi);
+        const int64_t lack = steady - live_pages(*m, kv.second, gi);
         if (lack > 0) need += lack;
       }
     }
@@ -183,7 +197,8 @@ int cm_reserve(void* h, int64_t id, int64_t new_len) {
 
 // Gives back, in windowed groups, the pages that no token at position >= computed_len can see any more:
 // a query at position p sees keys p - W + 1 .. p, so every key below computed_len - W + 1 is dead; with chunks of W
-// positions the next token sees its chunk from (computed_len / W) * W on.
+// positions the next token sees its chunk from (computed_len / W) * W on.  Pages that hold one of the first `keep` tokens
+// stay.
 // Returns the number of pages released.
 int cm_release_behind(void* h, int64_t id, int64_t computed_len) {
   Manager* m = static_cast<Manager*>(h);
@@ -198,7 +213,8 @@ int cm_release_behind(void* h, int64_t id, int64_t computed_len) {
     if (first_needed <= 0) continue;
     int64_t dead_blocks = first_needed / g.page_size;  // blocks wholly below first_needed
     if (dead_blocks > (int64_t)r.tables[gi].size()) dead_blocks = (int64_t)r.tables[gi].size();
-    for (int64_t b = r.first_live[gi]; b < dead_blocks; ++b) {
+    const int64_t kept = kept_blocks(g);
+    for (int64_t b = r.first_live[gi] > kept ? r.first_live[gi] : kept; b < dead_blocks; ++b) {
       const int32_t p = r.tables[gi][b];
       if (p >= 0) {
         g.in_use[p] = 0;

@@ -5,7 +5,7 @@
 // [max(0, p - window + 1), p] of that request, read through its block table, after this step's keys and values
 // have been written.  That one rule covers whole prompts, portions of prompts and single decoded tokens
 // (bottom-right aligned causal mask, csrc/kernels/mask.h:171-172 of the reference).
-// Keys are visited in chunks of 64 starting at the first visible key, so the order of every reduction depends
+// Keys are visited in chunks of 64 starting at the first visible one, so the order of every reduction depends
 // only on (p, window): the result for a token does not depend on how the step was cut or batched.
 // Online softmax in float32 (csrc/kernels/softmax.h:128-186 of the reference); query head h reads KV head
 // h / (nh / nkv) (csrc/kernels/flash_fwd_kernel.h:593).  With slopes (one per query head) the score of key j for the
@@ -13,7 +13,9 @@
 // slopes too: csrc/kernels/mask.h:155-157, 179-186; its Llama passes none).
 // With chunk > 0 the token at p sees only the keys of its own chunk of positions, [(p / chunk) * chunk, p]
 // (chunks count from position 0 of the request).  With sinks (one float32 per query head) the softmax denominator
-// also holds exp(sinks[h]): a weight that belongs to no key and carries no value.
+// also holds exp(sinks[h]): a weight that belongs to no key and carries no value.  With keep > 0 a token whose window has
+// moved on also sees the first `keep` keys of its request, visited before those of the window.  Values may have another
+// number of columns (vd) than keys (hd).
 #include "common.h"
 #include "cache_layout.h"
 
@@ -28,7 +30,8 @@ paged_attention_generic_kernel(const TQ* __restrict__ q, int q_stride, const TC*
                                const int32_t* __restrict__ block_tables, int max_blocks,
                                const int32_t* __restrict__ token_seq, const int32_t* __restrict__ positions,
                                float scale, int window, int page_size, int nh, int nkv, int hd,
-                               const float* __restrict__ slopes, int chunk, const float* __restrict__ sinks) {
+                               const float* __restrict__ slopes, int chunk, const float* __restrict__ sinks, int keep,
+                               int vd) {
   __shared__ float qs[kMaxHead];
   __shared__ float ps[kWave];
   __shared__ int32_t pg[kWave];
@@ -40,6 +43,8 @@ paged_attention_generic_kernel(const TQ* __restrict__ q, int q_stride, const TC*
   const int32_t* table = block_tables + (size_t)s * max_blocks;
   int first = (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
   if (chunk > 0 && (p / chunk) * chunk > first) first = (p / chunk) * chunk;
+  // visited keys, counted: the kept ones, then first .. p
+  const int kept = keep < first ? keep : first, visits = kept + p - first + 1;
   const float slope = slopes ? slopes[h] : 0.f;
 
   for (int d = lane; d < hd; d += kWave) qs[d] = to_f32(q[(size_t)t * q_stride + (size_t)h * hd + d]);
@@ -48,8 +53,8 @@ paged_attention_generic_kernel(const TQ* __restrict__ q, int q_stride, const TC*
   float m = -INFINITY, l = 0.f;
   float acc[kMaxHead / kWave] = {0.f, 0.f, 0.f, 0.f};
 
-  for (int base = first; base <= p; base += kWave) {
-    const int j = base + lane;
+  for (int base = 0; base < visits; base += kWave) {
+    const int j = base + lane < kept ? base + lane : base + lane - kept + first;
     const bool valid = j <= p;
     float sc = -INFINITY;
     int page = 0, off = 0;
@@ -76,15 +81,15 @@ paged_attention_generic_kernel(const TQ* __restrict__ q, int q_stride, const TC*
     pg[lane] = page;
     of[lane] = off;
     __syncthreads();
-    const int n = (p - base + 1 < kWave) ? p - base + 1 : kWave;
+    const int n = visits - base < kWave ? visits - base : kWave;
 #pragma unroll
     for (int i = 0; i < kMaxHead / kWave; ++i) {
       const int d = lane + i * kWave;
-      if (d < hd) {
+      if (d < vd) {
         float a = acc[i] * corr;
         for (int jj = 0; jj < n; ++jj)
-          a += ps[jj] * to_f32(vcache[((size_t)pg[jj] * nkv + kvh) * hd * page_size +
-                                      value_offset(d, of[jj], hd, page_size)]);
+          a += ps[jj] * to_f32(vcache[((size_t)pg[jj] * nkv + kvh) * vd * page_size +
+                                      value_offset(d, of[jj], vd, page_size)]);
         acc[i] = a;
       }
     }
@@ -102,7 +107,7 @@ paged_attention_generic_kernel(const TQ* __restrict__ q, int q_stride, const TC*
 #pragma unroll
   for (int i = 0; i < kMaxHead / kWave; ++i) {
     const int d = lane + i * kWave;
-    if (d < hd) out[(size_t)t * out_stride + (size_t)h * hd + d] = from_f32<TQ>(acc[i] * inv);
+    if (d < vd) out[(size_t)t * out_stride + (size_t)h * vd + d] = from_f32<TQ>(acc[i] * inv);
   }
 }
 
@@ -111,15 +116,15 @@ extern "C" int atoma_paged_attention_generic(const void* q, int q_stride, const 
                                              const int32_t* block_tables, int max_blocks, const int32_t* token_seq,
                                              const int32_t* positions, float scale, int window, int page_size,
                                              int n_tokens, int nh, int nkv, int hd, const float* slopes,
-                                             int chunk, const float* sinks, hipStream_t stream) {
+                                             int chunk, const float* sinks, int keep, int vd, hipStream_t stream) {
   if (n_tokens <= 0) return 0;
-  if (hd <= 0 || hd > kMaxHead || nkv <= 0 || nh % nkv || page_size <= 0 || max_blocks <= 0 || nh > 65535)
+  if (hd <= 0 || hd > kMaxHead || vd <= 0 || vd > kMaxHead || keep < 0 || nkv <= 0 || nh % nkv || page_size <= 0 || max_blocks <= 0 || nh > 65535)
     return ATOMA_ERR_SHAPE;
   dim3 grid(n_tokens, nh), block(kWave);
 #define ATOMA_ATTN(TQ, TC)                                                                                       \
   hipLaunchKernelGGL((paged_attention_generic_kernel<TQ, TC>), grid, block, 0, stream, (const TQ*)q, q_stride, \
                      (const TC*)kcache, (const TC*)vcache, (TQ*)out, out_stride, block_tables, max_blocks,      \
-                     token_seq, positions, scale, window, page_size, nh, nkv, hd, slopes, chunk, sinks)
+                     token_seq, positions, scale, window, page_size, nh, nkv, hd, slopes, chunk, sinks, keep, vd)
   if (act_dtype == kF32 && cache_dtype == kF32) ATOMA_ATTN(float, float);
   else if (act_dtype == kBF16 && cache_dtype == kBF16) ATOMA_ATTN(bf16_t, bf16_t);
   else if (act_dtype == kF32 && cache_dtype == kBF16) ATOMA_ATTN(float, bf16_t);

@@ -1,6 +1,7 @@
 // bfloat16 attention over the paged cache on the matrix cores, for prompts, portions and decoded tokens alike.
 // Compiled once per head size and page size: -DATOMA_HD=<multiple of 16, at most 256>, -DATOMA_PAGE=<tokens a page, a
-// multiple of 16; 16 if not given>.
+// multiple of 16; 16 if not given>; optionally -DATOMA_VD=<columns of a value head, a multiple of 16; ATOMA_HD if not
+// given> and -DATOMA_BIASED, for scores with a bias by distance and for windows that keep a request's first keys.
 //
 // Work is cut on the host into tasks, one per wave: 32 query rows against a range of keys.  A row is a
 // (token, query head) pair of one request and one KV head: row r of a tile is head r / qt, token tok0 + r % qt,
@@ -26,6 +27,12 @@
 //   O^T[d, row] += V^T[d, key] . P^T[key, row]  S^T's accumulator layout is already the B operand layout, so
 //                                             P goes from registers to the MFMA as bfloat16 without a
 //                                             transpose, and V^T is how the cache stores values.
+//
+// ATOMA_BIASED: the score of key j for the row at p gains slopes[head] * (j - p), and a row with a window also sees the
+// first `keep` keys of its request.  Between those keys and its window a tile leaves a gap of whole blocks out of its
+// walk: with keep_end = keep rounded up to 32 and lo the window's first key of the tile's first token rounded down to
+// 32, the walk's block at kb stands for the keys from kb on below keep_end, and from kb + gap on beyond, gap = lo -
+// keep_end where that is positive, else 0.  k_begin and k_end of such a task count along the walk.
 #include "common.h"
 
 using namespace atoma;
@@ -36,8 +43,18 @@ using namespace atoma;
 
 constexpr int HD = ATOMA_HD;
 static_assert(HD % 16 == 0 && HD >= 16 && HD <= 256, "head size must be a multiple of 16 up to 256");
+#ifndef ATOMA_VD
+#define ATOMA_VD ATOMA_HD
+#endif
+constexpr int VD = ATOMA_VD;           // columns of a value head
+static_assert(VD % 16 == 0 && VD >= 16 && VD <= 256, "value size must be a multiple of 16 up to 256");
+#ifdef ATOMA_BIASED
+constexpr bool BIASED = true;
+#else
+constexpr bool BIASED = false;
+#endif
 constexpr int KSTEPS = HD / 16;        // MFMA steps over the head dimension for S
-constexpr int DTILES = (HD + 31) / 32; // 32-row tiles of O^T
+constexpr int DTILES = (VD + 31) / 32; // 32-row tiles of O^T
 #ifndef ATOMA_PAGE
 #define ATOMA_PAGE 16
 #endif
@@ -113,7 +130,7 @@ template <int BATCH>
 __device__ __forceinline__ void merge_parts(const float* __restrict__ part_o, const float* __restrict__ part_lse,
                                             uint16_t* __restrict__ out, int out_stride, const Task& comb, int kvh,
                                             int nh, int nkv, int lane, const float* __restrict__ sinks) {
-  constexpr int Q = HD / 4;                        // pieces of four values in a row
+  constexpr int Q = VD / 4;                        // pieces of four values in a row
   const int g = nh / nkv;
   const size_t part_stride = (size_t)nkv * 32;     // rows between two parts of the same (KV head, row)
   const size_t base0 = ((size_t)comb.dest * nkv + kvh) * 32;
@@ -124,7 +141,7 @@ __device__ __forceinline__ void merge_parts(const float* __restrict__ part_o, co
     const int hq = r / comb.qt, tok = comb.tok0 + r % comb.qt;
     if (hq >= g || tok >= comb.count) continue;
     const float* pl = part_lse + base0 + c;
-    const float* po = part_o + (base0 + c) * HD + d;
+    const float* po = part_o + (base0 + c) * VD + d;
     float m = -INFINITY, wsum = 0.f;
     float4 acc = make_float4(0.f, 0.f, 0.f, 0.f);
     for (int s0 = 0; s0 < n_parts; s0 += BATCH) {
@@ -134,7 +151,7 @@ __device__ __forceinline__ void merge_parts(const float* __restrict__ part_o, co
       for (int u = 0; u < BATCH; ++u) {
         const int sp = s0 + u < n_parts ? s0 + u : n_parts - 1;
         ls[u] = load_through1(pl + (size_t)sp * part_stride);
-        v[u] = load_through(po + (size_t)sp * part_stride * HD);
+        v[u] = load_through(po + (size_t)sp * part_stride * VD);
       }
       float mb = m;
 #pragma unroll
@@ -165,7 +182,7 @@ __device__ __forceinline__ void merge_parts(const float* __restrict__ part_o, co
     uint2 pk;
     pk.x = (uint32_t)f32_to_bf16_bits(acc.x * inv) | ((uint32_t)f32_to_bf16_bits(acc.y * inv) << 16);
     pk.y = (uint32_t)f32_to_bf16_bits(acc.z * inv) | ((uint32_t)f32_to_bf16_bits(acc.w * inv) << 16);
-    *reinterpret_cast<uint2*>(out + (size_t)(comb.tok_base + tok) * out_stride + (size_t)(kvh * g + hq) * HD + d) = pk;
+    *reinterpret_cast<uint2*>(out + (size_t)(comb.tok_base + tok) * out_stride + (size_t)(kvh * g + hq) * VD + d) = pk;
   }
 }
 
@@ -191,7 +208,7 @@ attention_mfma_kernel(const Task* __restrict__ tasks, int n_tasks, int nkv, cons
                       const uint16_t* __restrict__ kcache, const uint16_t* __restrict__ vcache,
                       uint16_t* __restrict__ out, int out_stride, float* __restrict__ part_o,
                       float* __restrict__ part_lse, float scale, int32_t* __restrict__ counters,
-                      const float* __restrict__ sinks) {
+                      const float* __restrict__ sinks, int keep, const float* __restrict__ slopes) {
   // (the arguments come in the order in which a wave needs them: the first fourteen words, up to kcache, are in
   // scalar registers when the wave starts, the others are fetched from memory, a trip that the task record, the
   // queries, the page numbers and the first keys need not wait for)
@@ -238,6 +255,19 @@ attention_mfma_kernel(const Task* __restrict__ tasks, int n_tasks, int nkv, cons
   bool piece_on[RT];
 #pragma unroll
   for (int t = 0; t < RT; ++t) piece_on[t] = RT == 1 || __ballot(row_ok[t]) != 0;
+
+  // where the walk leaves keys out (the same for all tasks of a tile, and for all lanes)
+  int keep_end = 0, gap = 0;
+  if constexpr (BIASED) {
+    keep_end = (keep + 31) & ~31;
+    const int lo = (__builtin_amdgcn_readfirstlane(task.pos0 + task.tok0) - window + 1) & ~31;
+    gap = (keep > 0 && window > 0 && lo > keep_end) ? lo - keep_end : 0;
+  }
+  auto key_of = [&](int kb) { return BIASED && kb >= keep_end ? kb + gap : kb; };
+  // the rows' slopes, in the units of the exponentials
+  float sl2[RT];
+#pragma unroll
+  for (int t = 0; t < RT; ++t) sl2[t] = (BIASED && slopes != nullptr) ? slopes[head[t]] * kLog2e : 0.f;
 
   // page numbers: lane i asks for page (kb / PAGE + i) of the task's request; lanes 0 and 1 hold the pages that the two
   // runs of 16 keys of the block at kb may lie in (with pages of 32, 64, ... tokens both in lane 0's).  Asked for at the
@@ -293,19 +323,19 @@ attention_mfma_kernel(const Task* __restrict__ tasks, int n_tasks, int nkv, cons
       for (int i = 0; i < 16; ++i) o[t][dt][i] = 0.f;
   }
 
-  const size_t kv_head_stride = (size_t)PAGE * HD;            // one (page, head) tile
-  const size_t page_stride = (size_t)nkv * kv_head_stride;
+  const size_t k_head_stride = (size_t)PAGE * HD, v_head_stride = (size_t)PAGE * VD;      // one (page, head) tile
+  const size_t k_page_stride = (size_t)nkv * k_head_stride, v_page_stride = (size_t)nkv * v_head_stride;
 
   // Page numbers are the same in all lanes, so a tile's address is scalar arithmetic and a lane adds its own
   // offset, which never changes: tile order (cache_layout.h): keys: for each 16 columns, the 8-column pieces of all 16
   // tokens side by side; values: this lane's eight key slots of column d are one 16-byte piece.
-  const uint16_t* const k_tiles = kcache + (size_t)kvh * kv_head_stride;
-  const uint16_t* const v_tiles = vcache + (size_t)kvh * kv_head_stride;
+  const uint16_t* const k_tiles = kcache + (size_t)kvh * k_head_stride;
+  const uint16_t* const v_tiles = vcache + (size_t)kvh * v_head_stride;
   const uint32_t k_lane = (uint32_t)(hg * PAGE + (c & 15)) * 8;
   auto load_keys = [&](int kb, int p0, int p1, bf16x8* kf) {
     // (a key's 8-column pieces lie PAGE * 8 elements apart, the tokens of a piece side by side: a run starts 16 * 8 in)
-    const uint16_t* const t0 = k_tiles + (size_t)__builtin_amdgcn_readfirstlane(p0) * page_stride + run_of(kb) * 128;
-    const uint16_t* const t1 = k_tiles + (size_t)__builtin_amdgcn_readfirstlane(p1) * page_stride + run_of(kb + 16) * 128;
+    const uint16_t* const t0 = k_tiles + (size_t)__builtin_amdgcn_readfirstlane(p0) * k_page_stride + run_of(kb) * 128;
+    const uint16_t* const t1 = k_tiles + (size_t)__builtin_amdgcn_readfirstlane(p1) * k_page_stride + run_of(kb + 16) * 128;
     const uint16_t* kp = ((c < 16) ? t0 : t1) + k_lane;
 #pragma unroll
     for (int st = 0; st < KSTEPS; ++st) kf[st] = *reinterpret_cast<const bf16x8*>(kp + st * (2 * PAGE * 8));
@@ -314,14 +344,14 @@ attention_mfma_kernel(const Task* __restrict__ tasks, int n_tasks, int nkv, cons
   auto load_vals = [&](int kb, int p0, int p1, bf16x8 (*vf)[DTILES]) {
 #pragma unroll
     for (int j = 0; j < 2; ++j) {
-      const uint16_t* const tile = v_tiles + (size_t)__builtin_amdgcn_readfirstlane(j ? p1 : p0) * page_stride +
-                                   run_of(kb + 16 * j) * (16 * HD);
+      const uint16_t* const tile = v_tiles + (size_t)__builtin_amdgcn_readfirstlane(j ? p1 : p0) * v_page_stride +
+                                   run_of(kb + 16 * j) * (16 * VD);
 #pragma unroll
       for (int dt = 0; dt < DTILES; ++dt) {
         const int d = dt * 32 + c;
-        if (HD % 32 == 0 || d < HD) {
-          constexpr int last_rows = HD % 32 == 0 ? 32 : HD % 32;
-          const int rows = (HD % 32 == 0 || dt < DTILES - 1) ? 32 : last_rows;
+        if (VD % 32 == 0 || d < VD) {
+          constexpr int last_rows = VD % 32 == 0 ? 32 : VD % 32;
+          const int rows = (VD % 32 == 0 || dt < DTILES - 1) ? 32 : last_rows;
           const uint32_t v_lane = (uint32_t)(dt * 512 + (hg * rows + c) * 8);
           vf[j][dt] = *reinterpret_cast<const bf16x8*>(tile + v_lane);
         } else {
@@ -344,16 +374,18 @@ attention_mfma_kernel(const Task* __restrict__ tasks, int n_tasks, int nkv, cons
   bf16x8 vf[2][DTILES];
   int p0 = 0, p1 = 0;
   if (k_first < k_end) {
-    const int pw = page_window(k_first);
+    const int rk = key_of(k_first);
+    const int pw = page_window(rk);
     p0 = __builtin_amdgcn_readlane(pw, 0);
-    p1 = __builtin_amdgcn_readlane(pw, second_lane(k_first));
-    load_keys(k_first, p0, p1, kf);
+    p1 = __builtin_amdgcn_readlane(pw, second_lane(rk));
+    load_keys(rk, p0, p1, kf);
   }
   auto turn = [&](int kb, auto more) {
     constexpr bool MORE = decltype(more)::value;
     int pw = 0;
-    if constexpr (MORE) pw = page_window(kb + STRIDE);
-    load_vals(kb, p0, p1, vf);
+    const int rk = key_of(kb);        // the block's first key
+    if constexpr (MORE) pw = page_window(key_of(kb + STRIDE));
+    load_vals(rk, p0, p1, vf);
     // (no instruction: it keeps the compiler from moving these loads down to where their values are used)
     asm volatile("" ::: "memory");
     // S^T = K Q^T, for each piece of rows against the same fragments of the keys
@@ -369,22 +401,39 @@ attention_mfma_kernel(const Task* __restrict__ tasks, int n_tasks, int nkv, cons
       }
     }
     if constexpr (MORE) {
+      const int nk = key_of(kb + STRIDE);
       p0 = __builtin_amdgcn_readlane(pw, 0);
-      p1 = __builtin_amdgcn_readlane(pw, second_lane(kb + STRIDE));
-      load_keys(kb + STRIDE, p0, p1, kf);
+      p1 = __builtin_amdgcn_readlane(pw, second_lane(nk));
+      load_keys(nk, p0, p1, kf);
       asm volatile("" ::: "memory");
     }
 
     // Online softmax; accumulator element i is key kb + (i/4)*8 + hg*4 + i%4.  The running maximum is kept in
     // units of the scaled score (score * scale * log2 e), so one fused multiply-add feeds exp2.  Only blocks
     // that touch a row's own position, the window's edge or the end of the key range need the mask.
-    const bool edge = kb + 31 > p_lo || kb < lo_hi || kb + 32 > k_end;
+    const bool edge = rk + 31 > p_lo || rk < lo_hi || kb + 32 > k_end;
 #pragma unroll
     for (int t = 0; t < RT; ++t) {
       if (!piece_on[t]) continue;
       float sv[16];
       float bmax = -INFINITY;
-      if (edge) {
+      if constexpr (BIASED) {
+        // (a score is then in the units of the exponentials: times scale and log2 e, with its bias)
+        const float at = sl2[t] * (float)(rk + hg * 4 - p_row[t]);
+#pragma unroll
+        for (int i = 0; i < 16; ++i)
+          sv[i] = fmaf(s[t][i], sc2, fmaf(sl2[t], (float)((i >> 2) * 8 + (i & 3)), at));
+        if (edge) {
+#pragma unroll
+          for (int i = 0; i < 16; ++i) {
+            const int off = (i >> 2) * 8 + hg * 4 + (i & 3), key = rk + off;
+            const bool ok = key <= p_row[t] && (key >= lo_row[t] || key < keep) && kb + off < k_end;
+            sv[i] = ok ? sv[i] : -INFINITY;
+          }
+        }
+#pragma unroll
+        for (int i = 0; i < 16; ++i) bmax = fmaxf(bmax, sv[i]);
+      } else if (edge) {
 #pragma unroll
         for (int i = 0; i < 16; ++i) {
           const int key = kb + (i >> 2) * 8 + hg * 4 + (i & 3);
@@ -399,7 +448,8 @@ attention_mfma_kernel(const Task* __restrict__ tasks, int n_tasks, int nkv, cons
           bmax = fmaxf(bmax, sv[i]);
         }
       }
-      bmax = fmaxf(bmax, from_other_half(bmax, hg != 0)) * sc2;
+      bmax = fmaxf(bmax, from_other_half(bmax, hg != 0));
+      if constexpr (!BIASED) bmax *= sc2;
       // The reference point m of a row's exponentials follows its maximum only in jumps: as long as no row of the
       // wave has grown by more than kSlack (in powers of two) beyond its m, m stays, the weights may exceed one (by
       // at most 2^kSlack, nothing to float32 sums or to bfloat16 weights, whose precision is relative) and the
@@ -419,7 +469,7 @@ attention_mfma_kernel(const Task* __restrict__ tasks, int n_tasks, int nkv, cons
       float psum = 0.f;
 #pragma unroll
       for (int i = 0; i < 16; ++i) {
-        sv[i] = __builtin_amdgcn_exp2f(fmaf(sv[i], sc2, -m_use));
+        sv[i] = __builtin_amdgcn_exp2f(BIASED ? sv[i] - m_use : fmaf(sv[i], sc2, -m_use));
         psum += sv[i];
       }
       l[t] += psum;      // this lane's half of the row's sum; the halves meet after the last block
@@ -500,13 +550,13 @@ attention_mfma_kernel(const Task* __restrict__ tasks, int n_tasks, int nkv, cons
           for (int i = 0; i < 16; ++i) o[t][dt][i] *= corr;
       }
       const float inv = l[t] > 0.f ? 1.0f / l[t] : 0.f;
-      uint16_t* op = out + (size_t)trow[t] * out_stride + (size_t)head[t] * HD;
+      uint16_t* op = out + (size_t)trow[t] * out_stride + (size_t)head[t] * VD;
 #pragma unroll
       for (int dt = 0; dt < DTILES; ++dt)
 #pragma unroll
         for (int q4 = 0; q4 < 4; ++q4) {
           const int d = dt * 32 + q4 * 8 + hg * 4;
-          if (HD % 32 == 0 || d < HD) {
+          if (VD % 32 == 0 || d < VD) {
             uint2 v;
             v.x = (uint32_t)f32_to_bf16_bits(o[t][dt][q4 * 4 + 0] * inv) |
                   ((uint32_t)f32_to_bf16_bits(o[t][dt][q4 * 4 + 1] * inv) << 16);
@@ -520,14 +570,14 @@ attention_mfma_kernel(const Task* __restrict__ tasks, int n_tasks, int nkv, cons
     // a partial result is one piece of 32 rows (the host gives such tasks one piece, whatever RT is);
     // rows that are not live are never read by the merge (their log-sum-exp is, and says -inf)
     const float inv = l[0] > 0.f ? 1.0f / l[0] : 0.f;
-    float* po = part_o + (((size_t)task.dest * nkv + kvh) * 32 + c) * HD;
+    float* po = part_o + (((size_t)task.dest * nkv + kvh) * 32 + c) * VD;
     const bool merge_here = counters != nullptr;
 #pragma unroll
     for (int dt = 0; dt < DTILES; ++dt)
 #pragma unroll
       for (int q4 = 0; q4 < 4; ++q4) {
         const int d = dt * 32 + q4 * 8 + hg * 4;
-        if (row_ok[0] && (HD % 32 == 0 || d < HD)) {
+        if (row_ok[0] && (VD % 32 == 0 || d < VD)) {
           float4 v = make_float4(o[0][dt][q4 * 4 + 0] * inv, o[0][dt][q4 * 4 + 1] * inv, o[0][dt][q4 * 4 + 2] * inv,
                                  o[0][dt][q4 * 4 + 3] * inv);
           if (merge_here) store_through(po + d, v);
@@ -568,7 +618,7 @@ attention_mfma_kernel(const Task* __restrict__ tasks, int n_tasks, int nkv, cons
 // to memory it saves the launch.
 // One block per (combine task, KV head).  The log-sum-exps of all parts are first brought into LDS by all
 // threads at once and turned into weights there; then the valid rows of the task (group x tokens, at most 32)
-// times HD output values are spread over the 256 threads, and each adds its parts in order of their index with
+// times VD output values are spread over the 256 threads, and each adds its parts in order of their index with
 // eight loads in flight.
 constexpr int kCombineParts = 128;   // parts whose weights fit in LDS at once; more are merged in rounds
 
@@ -605,10 +655,10 @@ attention_combine_kernel(const float* __restrict__ part_o, const float* __restri
     __syncthreads();
   }
 
-  float acc[(32 * HD + 255) / 256];
-  float wsum[(32 * HD + 255) / 256];
+  float acc[(32 * VD + 255) / 256];
+  float wsum[(32 * VD + 255) / 256];
 #pragma unroll
-  for (int i = 0; i < (32 * HD + 255) / 256; ++i) acc[i] = wsum[i] = 0.f;
+  for (int i = 0; i < (32 * VD + 255) / 256; ++i) acc[i] = wsum[i] = 0.f;
 
   for (int p0 = 0; p0 < task.n_parts; p0 += kCombineParts) {
     const int np = task.n_parts - p0 < kCombineParts ? task.n_parts - p0 : kCombineParts;
@@ -619,18 +669,18 @@ attention_combine_kernel(const float* __restrict__ part_o, const float* __restri
     }
     __syncthreads();
 #pragma unroll
-    for (int it = 0; it < (32 * HD + 255) / 256; ++it) {
+    for (int it = 0; it < (32 * VD + 255) / 256; ++it) {
       const int idx = tid + it * 256;
-      const int c = idx / HD, d = idx % HD;
+      const int c = idx / VD, d = idx % VD;
       const int r = task.row0 + c;
       const int hq = r / task.qt, tok = task.tok0 + r % task.qt;
-      if (idx >= 32 * HD || hq >= g || tok >= count) continue;
-      const float* po = part_o + (base0 + (size_t)p0 * part_stride + c) * HD + d;
+      if (idx >= 32 * VD || hq >= g || tok >= count) continue;
+      const float* po = part_o + (base0 + (size_t)p0 * part_stride + c) * VD + d;
       int s = 0;
       for (; s + 8 <= np; s += 8) {
         float v[8];
 #pragma unroll
-        for (int u = 0; u < 8; ++u) v[u] = po[(size_t)(s + u) * part_stride * HD];
+        for (int u = 0; u < 8; ++u) v[u] = po[(size_t)(s + u) * part_stride * VD];
 #pragma unroll
         for (int u = 0; u < 8; ++u) {
           acc[it] += wts[s + u][c] * v[u];
@@ -638,20 +688,20 @@ attention_combine_kernel(const float* __restrict__ part_o, const float* __restri
         }
       }
       for (; s < np; ++s) {
-        acc[it] += wts[s][c] * po[(size_t)s * part_stride * HD];
+        acc[it] += wts[s][c] * po[(size_t)s * part_stride * VD];
         wsum[it] += wts[s][c];
       }
     }
   }
 #pragma unroll
-  for (int it = 0; it < (32 * HD + 255) / 256; ++it) {
+  for (int it = 0; it < (32 * VD + 255) / 256; ++it) {
     const int idx = tid + it * 256;
-    const int c = idx / HD, d = idx % HD;
+    const int c = idx / VD, d = idx % VD;
     const int r = task.row0 + c;
     const int hq = r / task.qt, tok = task.tok0 + r % task.qt;
-    if (idx >= 32 * HD || hq >= g || tok >= count) continue;
+    if (idx >= 32 * VD || hq >= g || tok >= count) continue;
     const float sink_w = sinks != nullptr ? __builtin_amdgcn_exp2f(sinks[kvh * g + hq] * kLog2e - row_max[c]) : 0.f;
-    out[(size_t)(tok_base + tok) * out_stride + (size_t)(kvh * g + hq) * HD + d] =
+    out[(size_t)(tok_base + tok) * out_stride + (size_t)(kvh * g + hq) * VD + d] =
         f32_to_bf16_bits(acc[it] / (wsum[it] + sink_w));
   }
 }
@@ -664,12 +714,12 @@ constexpr size_t kMerge4Bytes = (DTILES * 16 + 2) * 64 * 6 * sizeof(float);     
 constexpr size_t kMerge8Bytes = (DTILES * 16 + 2) * 64 * 7 * sizeof(float);
 // (heads beyond 192 columns: a wave's output alone is more than a hundred registers a lane, and with the eight waves of
 // a split workgroup a lane may have 256; such heads keep one wave a task and four waves a workgroup)
-constexpr bool kSplit2Fits = kMerge2Bytes <= kLdsBytes && HD <= 192;
-constexpr bool kSplit4Fits = kMerge4Bytes <= kLdsBytes;
-constexpr bool kSplit8Fits = kMerge8Bytes <= kLdsBytes;
+constexpr bool kSplit2Fits = kMerge2Bytes <= kLdsBytes && HD <= 192 && VD <= 192;
+constexpr bool kSplit4Fits = kMerge4Bytes <= kLdsBytes && HD <= 192;
+constexpr bool kSplit8Fits = kMerge8Bytes <= kLdsBytes && HD <= 192;
 // two pieces of rows a wave: where the accumulators of both fit the registers of eight waves a workgroup, and the
 // merge of two waves a task (twice as large) lets two workgroups share a CU
-constexpr bool kTwoPieces = HD <= 64;
+constexpr bool kTwoPieces = HD <= 64 && VD <= 64;
 
 // A kernel that wants more than 64 KB of LDS at launch must be told so once per device: every instance of the
 // template keeps, per device, whether it has been (a driver call per launch would sit on the path of every layer of
@@ -689,19 +739,23 @@ template <typename K> static int allow_lds(K kernel, size_t bytes) {
 }
 
 extern "C" int atoma_attention_mfma_head_size() { return HD; }
+extern "C" int atoma_attention_mfma_value_size() { return VD; }
+extern "C" int atoma_attention_mfma_biased() { return BIASED; }
 extern "C" int atoma_attention_mfma_page_size() { return PAGE; }
 extern "C" int atoma_attention_mfma_max_ksplit() { return kSplit8Fits ? 8 : kSplit2Fits ? 2 : 1; }
 extern "C" int atoma_attention_mfma_max_row_tiles() { return kTwoPieces ? 2 : 1; }
 
 // tasks: device array of n_tasks Task records (main kernel), followed by n_combine records of the row pieces whose
 // keys are cut into chunks.  counters: null, or n_combine * nkv zeros (left as zeros again): the attention kernel then
-// merges the chunks itself and the combine kernel does not run.
+// merges the chunks itself and the combine kernel does not run.  keep (keys of a request that a window never loses) and
+// slopes (null, or one float32 per query head) need a module compiled with ATOMA_BIASED.
 extern "C" int atoma_attention_mfma(const void* q, int q_stride, const void* kcache, const void* vcache, void* out,
                                     int out_stride, float* part_o, float* part_lse, const int32_t* tasks, int n_tasks,
                                     int n_combine, const int32_t* block_tables, int max_blocks, float scale,
                                     int window, int nh, int nkv, int ksplit, int row_tiles, int32_t* counters,
-                                    const float* sinks, hipStream_t stream) {
+                                    const float* sinks, int keep, const float* slopes, hipStream_t stream) {
   if (n_tasks <= 0) return 0;
+  if (keep < 0 || (keep > 0 && window <= 0) || (!BIASED && (keep > 0 || slopes != nullptr))) return ATOMA_ERR_SHAPE;
   // row_tiles: 1, or 2: the tasks that write the output cover 64 rows (Task::tiles says so), two waves a task
   if (row_tiles != 1 && !(row_tiles == 2 && kTwoPieces && ksplit == 2)) return ATOMA_ERR_SHAPE;
   if (nkv <= 0 || nh % nkv || nkv > 65535 || max_blocks <= 0 || (q_stride & 7) || (out_stride & 3) ||
@@ -718,11 +772,11 @@ extern "C" int atoma_attention_mfma(const void* q, int q_stride, const void* kca
                        dim3(64 * T * KS), BYTES,                                                                   \
                        stream, t, n_tasks, nkv, (const uint16_t*)q, q_stride, nh, block_tables, max_blocks,        \
                        window, (const uint16_t*)kcache, (const uint16_t*)vcache, (uint16_t*)out, out_stride,       \
-                       part_o, part_lse, scale, counters, sinks);                                                  \
+                       part_o, part_lse, scale, counters, sinks, keep, slopes);                                               \
   } while (0)
   // (wide heads keep one wave a task, see kSplit2Fits: with few tasks, as in a decode step over one shared key/value
   // head, a workgroup of four of them would leave most CUs without work, so each task gets a workgroup of its own)
-  if (ksplit == 1 && HD > 192 && (size_t)n_tasks * nkv <= 1024) ATOMA_ATTN(1, 1, 0);
+  if (ksplit == 1 && !kSplit2Fits && (size_t)n_tasks * nkv <= 1024) ATOMA_ATTN(1, 1, 0);
   else if (ksplit == 1) ATOMA_ATTN(4, 1, 0);
   else if (ksplit == 2 && row_tiles == 2) ATOMA_ATTN(4, 2, 2 * kMerge2Bytes, (kTwoPieces ? 2 : 1));
   else if (ksplit == 2 && kSplit2Fits) ATOMA_ATTN(4, (kSplit2Fits ? 2 : 1), kMerge2Bytes);

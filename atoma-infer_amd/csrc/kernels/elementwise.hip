@@ -47,6 +47,47 @@ __global__ void embed_kernel(const int32_t* __restrict__ tokens, const TW* __res
   for (int i = threadIdx.x; i < width; i += blockDim.x) out[dst + i] = to_f32(table[src + i]) * scale;
 }
 
+// The gather with a sinusoid of the position: out[t, c] = table[token[t], c] * scale + sin or cos (c even or odd) of
+// positions[t] * freq[c / 2].  The angle is reduced to one turn in float64, so it is exact to float32 at any position.
+template <typename TW>
+__global__ void __launch_bounds__(256)
+embed_sinusoid_kernel(const int32_t* __restrict__ tokens, const TW* __restrict__ table, float* __restrict__ out,
+                      const int32_t* __restrict__ positions, const double* __restrict__ freq, int width, int vocab,
+                      float scale) {
+  const int t = blockIdx.x;
+  const int token = tokens[t];
+  const bool ok = token >= 0 && token < vocab;
+  const double p = (double)positions[t];
+  const size_t dst = (size_t)t * width, src = (size_t)(ok ? token : 0) * width;
+  for (int i = threadIdx.x; 2 * i < width; i += 256) {
+    double turns = p * freq[i] * 0.15915494309189535;      // 1 / (2 pi)
+    turns -= rint(turns);
+    float s, c;
+    sincosf((float)(turns * 6.283185307179586), &s, &c);
+    const int col = 2 * i;
+    out[dst + col] = ok ? to_f32(table[src + col]) * scale + s : __int_as_float(0x7fc00000);
+    if (col + 1 < width) out[dst + col + 1] = ok ? to_f32(table[src + col + 1]) * scale + c : __int_as_float(0x7fc00000);
+  }
+}
+
+extern "C" int atoma_embed_sinusoid(const int32_t* tokens, const void* table, int table_dtype, float* out,
+                                    const int32_t* positions, const double* freq, int n_tokens, int width, int vocab,
+                                    float scale, hipStream_t stream) {
+  if (n_tokens <= 0) return 0;
+  if (width <= 0 || positions == nullptr || freq == nullptr) return ATOMA_ERR_SHAPE;
+  dim3 grid(n_tokens), block(256);
+  if (table_dtype == kF32)
+    hipLaunchKernelGGL(embed_sinusoid_kernel<float>, grid, block, 0, stream, tokens, (const float*)table, out, positions,
+                       freq, width, vocab, scale);
+  else if (table_dtype == kBF16)
+    hipLaunchKernelGGL(embed_sinusoid_kernel<bf16_t>, grid, block, 0, stream, tokens, (const bf16_t*)table, out, positions,
+                       freq, width, vocab, scale);
+  else
+    return ATOMA_ERR_DTYPE;
+  ATOMA_LAUNCH_CHECK();
+  return 0;
+}
+
 extern "C" int atoma_embed(const int32_t* tokens, const void* table, int table_dtype, float* out, int n_tokens,
                            int width, int vocab, float scale, hipStream_t stream) {
   if (n_tokens <= 0) return 0;

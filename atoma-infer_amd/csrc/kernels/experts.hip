@@ -4,7 +4,8 @@
 //                 experts with the largest score + correction[expert] (no correction: the score alone; the lower
 //                 index wins a tie) with their weights, score * scale (the correction chooses, it does not weigh),
 //                 or the experts with the largest logits, weighed by the softmax over the chosen logits alone (times
-//                 scale); logits may have a bias per expert.
+//                 scale); logits may have a bias per expert.  With groups (equal runs of neighbouring experts) a group's
+//                 score is that of its best expert, and only experts of the best groups_keep groups can be chosen;
 //                 A (token, choice) pair is a "slot", numbered token * top + choice;
 //   route_group   one workgroup: slots ordered by expert (perm), where each expert's slots start (offsets), and the
 //                 list of row tiles (expert, first place in perm) that the products below walk.  Which place a slot
@@ -24,14 +25,17 @@ using namespace atoma;
 
 constexpr int kTileM = 64, kTileN = 64, kStepK = 16;
 
+template <bool GROUPED>
 __global__ void __launch_bounds__(256)
 route_topk_kernel(const float* __restrict__ logits, int ld, int experts, int top, int32_t* __restrict__ ids,
                   float* __restrict__ weights, int n_tokens, int score, const float* __restrict__ correction,
-                  float scale, const float* __restrict__ bias) {
+                  float scale, const float* __restrict__ bias, int groups, int groups_keep) {
   // a wave a token; lane l holds experts l, l + 64, ...
   const int lane = threadIdx.x & 63;
-  const int t = blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (t >= n_tokens) return;
+  const int row = blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (!GROUPED && row >= n_tokens) return;
+  // (with groups all waves meet at barriers: one without a token works on the last one and stores nothing)
+  const int t = row < n_tokens ? row : n_tokens - 1;
   constexpr int PER = 16;      // experts <= 1024
   // sc: what chooses (score, plus the correction where there is one); wt: what weighs (the score alone)
   // score 0: sigmoid; 1: softmax over all experts; 2: the logits choose, softmax over the chosen ones (below)
@@ -64,6 +68,53 @@ route_topk_kernel(const float* __restrict__ logits, int ld, int experts, int top
   for (int j = 0; j < PER; ++j) {
     const int e = lane + j * 64;
     sc[j] = e < experts ? (correction != nullptr ? wt[j] + correction[e] : wt[j]) : -INFINITY;
+  }
+  if constexpr (GROUPED) {
+    // the scores of a wave's token in LDS, then its groups' scores over them; lane l holds groups l, l + 64, ...
+    __shared__ float table[4][1024];
+    float* const mine_t = table[threadIdx.x >> 6];
+    const int size = experts / groups;
+#pragma unroll
+    for (int j = 0; j < PER; ++j)
+      if (lane + j * 64 < experts) mine_t[lane + j * 64] = sc[j];
+    __syncthreads();
+    float gs[PER];
+#pragma unroll
+    for (int j = 0; j < PER; ++j) {
+      gs[j] = -INFINITY;
+      const int g = lane + j * 64;
+      if (g < groups)
+        for (int e = 0; e < size; ++e) gs[j] = fmaxf(gs[j], mine_t[g * size + e]);
+    }
+    __syncthreads();
+    // a kept group is marked where its scores were
+#pragma unroll
+    for (int j = 0; j < PER; ++j)
+      if (lane + j * 64 < groups) mine_t[lane + j * 64] = 0.f;
+    for (int c = 0; c < groups_keep; ++c) {
+      float best = -INFINITY;
+      int arg = 0x7fffffff;
+#pragma unroll
+      for (int j = 0; j < PER; ++j)
+        if (gs[j] > best) best = gs[j], arg = lane + j * 64;
+#pragma unroll
+      for (int off = 32; off > 0; off >>= 1) {
+        const float ob = __shfl_xor(best, off, 64);
+        const int oa = __shfl_xor(arg, off, 64);
+        if (ob > best || (ob == best && oa < arg)) best = ob, arg = oa;
+      }
+#pragma unroll
+      for (int j = 0; j < PER; ++j)
+        if (lane + j * 64 == arg) {
+          gs[j] = -INFINITY;
+          mine_t[arg] = 1.f;
+        }
+    }
+    __syncthreads();
+#pragma unroll
+    for (int j = 0; j < PER; ++j)
+      if (lane + j * 64 < experts && mine_t[(lane + j * 64) / size] == 0.f) sc[j] = -INFINITY;
+    if (row >= n_tokens) return;
   }
   for (int c = 0; c < top; ++c) {
     float best = -INFINITY, bw = 0.f;
@@ -424,13 +475,22 @@ extern "C" int atoma_expert_gemm_mfma(const void* a, const void* w, void* c, int
 
 extern "C" int atoma_route_topk(const float* logits, int ld, int experts, int top, int32_t* ids, float* weights,
                                 int n_tokens, int score, const float* correction, float scale, const float* bias,
-                                hipStream_t stream) {
+                                int groups, int groups_keep, hipStream_t stream) {
   if (n_tokens <= 0) return 0;
   if (experts <= 0 || experts > 1024 || top <= 0 || top > experts || ld < experts || score < 0 ||
       score > 2)
     return ATOMA_ERR_SHAPE;
-  hipLaunchKernelGGL(route_topk_kernel, dim3((n_tokens + 3) / 4), dim3(256), 0, stream, logits, ld, experts, top, ids,
-                     weights, n_tokens, score, correction, scale, bias);
+  // groups: 0 (none), or a number of equal runs of experts, of which groups_keep hold at least the top experts
+  if (groups < 0 || (groups > 0 && (experts % groups || groups_keep <= 0 || groups_keep > groups ||
+                                    groups_keep * (experts / groups) < top)))
+    return ATOMA_ERR_SHAPE;
+  const dim3 grid((n_tokens + 3) / 4), block(256);
+  if (groups > groups_keep)
+    hipLaunchKernelGGL(route_topk_kernel<true>, grid, block, 0, stream, logits, ld, experts, top, ids, weights, n_tokens,
+                       score, correction, scale, bias, groups, groups_keep);
+  else
+    hipLaunchKernelGGL(route_topk_kernel<false>, grid, block, 0, stream, logits, ld, experts, top, ids, weights, n_tokens,
+                       score, correction, scale, bias, 0, 0);
   ATOMA_LAUNCH_CHECK();
   return 0;
 }

@@ -6,7 +6,7 @@
 //   out   = resid / sqrt(mean(resid^2) + eps) * w_next            (optional, in the activation dtype)
 //
 // Without w_post the sum joins the stream as it is, resid += d: blocks whose sublayers read one norm and add their
-// outputs side by side.
+// outputs side by side.  A term of one plane whose plane stride is 0 is one row that joins every row of the stream.
 //
 // One workgroup a row; the row waits in LDS between the passes, so every operand is read once.  All statistics and
 // sums are float32.  The planes of a term are added in the order of their index and the terms in theirs, so a row's
@@ -19,9 +19,12 @@ struct Term {
   const void* data;      // [planes, T, width]
   int dtype;             // kF32 or kBF16
   int planes;
-  size_t plane_stride;   // elements between planes
+  size_t plane_stride;   // elements between planes; 0: one row for all
   float scale;
 };
+
+// where a term's elements for the stream's row at `base` begin
+__device__ __forceinline__ size_t row_of(const Term& t, size_t base) { return t.plane_stride == 0 ? 0 : base; }
 
 __device__ __forceinline__ float term_at(const Term& t, size_t idx) {
   float v = 0.f;
@@ -42,10 +45,11 @@ add_normed_kernel(float* __restrict__ resid, Term a, Term b, int n_terms, const 
   extern __shared__ float row[];
   __shared__ float scratch[4];
   const size_t base = (size_t)blockIdx.x * width;
+  const size_t base_a = row_of(a, base), base_b = row_of(b, base);
   float ss = 0.f;
   for (int i = threadIdx.x; i < width; i += 256) {
-    float d = term_at(a, base + i);
-    if (n_terms > 1) d += term_at(b, base + i);
+    float d = term_at(a, base_a + i);
+    if (n_terms > 1) d += term_at(b, base_b + i);
     row[i] = d;
     ss += d * d;
   }
@@ -142,11 +146,12 @@ add_normed_vec_kernel(float* __restrict__ resid, Term a, Term b, int n_terms, co
     const int c = threadIdx.x + j * 256;
     if (c < n4) x[j] = load4(resid + base + 4 * c);
   }
-  if (a.dtype == kF32) add_term<float, MAXJ>(d, a, base, n4);
-  else add_term<bf16_t, MAXJ>(d, a, base, n4);
+  const size_t base_a = row_of(a, base), base_b = row_of(b, base);
+  if (a.dtype == kF32) add_term<float, MAXJ>(d, a, base_a, n4);
+  else add_term<bf16_t, MAXJ>(d, a, base_a, n4);
   if (n_terms > 1) {
-    if (b.dtype == kF32) add_term<float, MAXJ>(d, b, base, n4);
-    else add_term<bf16_t, MAXJ>(d, b, base, n4);
+    if (b.dtype == kF32) add_term<float, MAXJ>(d, b, base_b, n4);
+    else add_term<bf16_t, MAXJ>(d, b, base_b, n4);
   }
   float ss = 0.f;
 #pragma unroll
@@ -212,6 +217,7 @@ extern "C" int atoma_add_normed(float* resid, const void* d0, int dtype0, int pl
   if (n_rows <= 0) return 0;
   if (width <= 0 || width > 16384 || d0 == nullptr || planes0 <= 0 || (d1 != nullptr && planes1 <= 0)) return ATOMA_ERR_SHAPE;
   if ((dtype0 != kF32 && dtype0 != kBF16) || (d1 != nullptr && dtype1 != kF32 && dtype1 != kBF16)) return ATOMA_ERR_DTYPE;
+  if ((stride0 == 0 && planes0 != 1) || (d1 != nullptr && stride1 == 0 && planes1 != 1)) return ATOMA_ERR_SHAPE;
   Term a{d0, dtype0, planes0, stride0, scale0}, b{d1, dtype1, planes1, stride1, scale1};
   const int n_terms = d1 != nullptr ? 2 : 1;
   const size_t lds = (size_t)width * sizeof(float);

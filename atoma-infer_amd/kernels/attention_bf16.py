@@ -3,6 +3,9 @@
 The mask is one integer everywhere here (``window``): w > 0 a window of the last w keys, -c < 0 chunks of c
 positions (a token sees the keys of its own chunk up to itself), 0 all keys; ``first_key`` states it.
 
+A window may keep a request's first keys beside the last w (``keep``); the tasks of such a layer count their keys along
+a walk that leaves the keys between out (``walk``), and run in the module that also takes scores biased by distance.
+
 ``try_attention`` runs ``attention_mfma.hip`` (compiled for the model's head size and the cache's page size on
 first use) when the cache's pages hold a multiple of 16 tokens; otherwise it returns False and the caller runs the
 general kernel.
@@ -31,7 +34,7 @@ SPLIT_MAX_TOKENS = 16  # entries with at most this many tokens may be split alon
 SPLIT_MIN_KEYS = 2 * CHUNK
 SPLIT_WAVES_MIN_KEYS = 128   # a task of at least this many keys is walked by two waves, every other block each
 FOUR_WAVES_MIN_KEYS = 256    # ... by four, where the launch leaves half of the GPU idle (see build_tasks)
-_libs: Dict[Tuple[int, int], ctypes.CDLL] = {}
+_libs: Dict[tuple, ctypes.CDLL] = {}
 
 
 def page_ok(page_size: int) -> bool:
@@ -40,43 +43,53 @@ def page_ok(page_size: int) -> bool:
     return page_size >= 16 and page_size % 16 == 0
 
 
-def module_name(hd: int, page: int = PAGE) -> str:
-    return f"attention_hd{hd}" if page == PAGE else f"attention_hd{hd}_page{page}"
+def module_name(hd: int, page: int = PAGE, vd: Optional[int] = None, biased: bool = False) -> str:
+    """``vd``: columns of a value head where they differ from a key head's; ``biased``: scores with a bias by distance,
+    and windows that keep a request's first keys."""
+    return (f"attention_hd{hd}" + (f"_vd{vd}" if vd not in (None, hd) else "") + ("_biased" if biased else "")
+            + (f"_page{page}" if page != PAGE else ""))
 
 
-def module_defines(hd: int, page: int = PAGE) -> Tuple[str, ...]:
-    return (f"ATOMA_HD={hd}",) if page == PAGE else (f"ATOMA_HD={hd}", f"ATOMA_PAGE={page}")
+def module_defines(hd: int, page: int = PAGE, vd: Optional[int] = None, biased: bool = False) -> Tuple[str, ...]:
+    return ((f"ATOMA_HD={hd}",) + ((f"ATOMA_VD={vd}",) if vd not in (None, hd) else ())
+            + (("ATOMA_BIASED",) if biased else ()) + ((f"ATOMA_PAGE={page}",) if page != PAGE else ()))
 
 
-def lib(hd: int, force_build: bool = False, page: int = PAGE) -> ctypes.CDLL:
-    key = (hd, page)
+def lib(hd: int, force_build: bool = False, page: int = PAGE, vd: Optional[int] = None, biased: bool = False) -> ctypes.CDLL:
+    vd = hd if vd is None else vd
+    key = (hd, page, vd, bool(biased))
     if key not in _libs or force_build:
-        _libs[key] = load_hip_module(module_name(hd, page), ("attention_mfma.hip",), module_defines(hd, page),
-                                     force_build=force_build)
+        _libs[key] = load_hip_module(module_name(hd, page, vd, biased), ("attention_mfma.hip",),
+                                     module_defines(hd, page, vd, biased), force_build=force_build)
         assert _libs[key].atoma_attention_mfma_head_size() == hd
+        assert _libs[key].atoma_attention_mfma_value_size() == vd
+        assert bool(_libs[key].atoma_attention_mfma_biased()) == bool(biased)
         assert _libs[key].atoma_attention_mfma_page_size() == page
-        assert _libs[key].atoma_attention_mfma_max_ksplit() == max_waves_for(hd)
-        assert _libs[key].atoma_attention_mfma_max_row_tiles() == max_row_tiles_for(hd)
+        assert _libs[key].atoma_attention_mfma_max_ksplit() == max_waves_for(hd, vd)
+        assert _libs[key].atoma_attention_mfma_max_row_tiles() == max_row_tiles_for(hd, vd)
     return _libs[key]
 
 
-def max_waves_for(hd: int) -> int:
-    """Waves that may share a task for this head size: their merge must fit into the 160 KB of LDS of a CU (the
-    kernel module says the same: ``atoma_attention_mfma_max_ksplit``)."""
-    per_lane = -(-hd // 32) * 16 + 2
+def max_waves_for(hd: int, vd: Optional[int] = None) -> int:
+    """Waves that may share a task for this head size (and value size): their merge must fit into the 160 KB of LDS of
+    a CU (the kernel module says the same: ``atoma_attention_mfma_max_ksplit``)."""
+    vd = hd if vd is None else vd
+    per_lane = -(-vd // 32) * 16 + 2
+    # (beyond 192 columns a wave's operands alone fill the registers that a lane of an eight-wave workgroup may have)
+    if max(hd, vd) > 192:
+        return 1
     if per_lane * 64 * 7 * 4 <= 160 * 1024:
         return 8
-    # (beyond 192 columns a wave's output alone fills the registers that a lane of an eight-wave workgroup may have)
-    return 2 if per_lane * 64 * 4 * 4 <= 160 * 1024 and hd <= 192 else 1
+    return 2 if per_lane * 64 * 4 * 4 <= 160 * 1024 else 1
 
 
 TWO_PIECES_MIN_KEYS = 16384     # keys from which on a wave of a prompt step works on two pieces of rows
 
 
-def max_row_tiles_for(hd: int) -> int:
+def max_row_tiles_for(hd: int, vd: Optional[int] = None) -> int:
     """Pieces of 32 rows that a wave of a prompt step may work on against the same keys (the kernel module says the
     same: ``atoma_attention_mfma_max_row_tiles``): two where the accumulators of both fit a wave's registers."""
-    return 2 if hd <= 64 else 1
+    return 2 if max(hd, vd or hd) <= 64 else 1
 
 
 # (request, KV head) pairs from which on a decoded token's keys are not cut into chunks: measured on MI355X (256 CUs),
@@ -232,9 +245,30 @@ def first_key(pos, window: int):
     return pos * 0
 
 
-def _chunk_slots(bucket_keys: int, chunk: int, window: int) -> int:
+def walk(first_pos, k_end, window: int, keep: int):
+    """(first key, end) of the keys that a tile of tokens from position ``first_pos`` on walks, its last token seeing keys
+    below ``k_end``, in whole blocks of 32 at the beginning.  Without ``keep`` these are key numbers.  With it the walk
+    begins at the request's first key, leaves out the whole blocks between the kept keys and the window of the tile's
+    first token, and counts on (the kernel turns its place in the walk into the key the same way)."""
+    lo = first_key(first_pos, window)
+    lo32 = (lo // 32) * 32
+    if not keep:
+        return lo32, k_end
+    keep_end = -(-keep // 32) * 32
+    return lo32 * 0, k_end - np.maximum(0, lo32 - keep_end)
+
+
+def _most_walked(bucket_keys: int, window: int, keep: int) -> int:
+    """The longest walk of a decoded token below ``bucket_keys`` keys behind a window that keeps ``keep`` keys."""
+    return min(bucket_keys, window + 31 + -(-keep // 32) * 32)
+
+
+def _chunk_slots(bucket_keys: int, chunk: int, window: int, keep: int = 0) -> int:
     """Partial results that a decoded token of a graph's bucket owns: one per chunk of the bucket's keys, or, with
-    a window, per chunk that a window can touch wherever it lies (its first chunk is then slot 0)."""
+    a window, per chunk that a window can touch wherever it lies (its first chunk is then slot 0), or, where the walk
+    begins at the request's first key, per chunk of the longest walk."""
+    if keep:
+        return -(-_most_walked(bucket_keys, window, keep) // chunk)
     slots = -(-bucket_keys // chunk)
     if window != 0:
         slots = min(slots, -(-abs(window) // chunk) + 1)
@@ -244,7 +278,8 @@ def _chunk_slots(bucket_keys: int, chunk: int, window: int) -> int:
 _NULL_TASK = np.asarray((-1, 0, 1, 0, 0, 0, -1, 0, 0, 0, 0, 0), dtype=np.int32)
 
 
-def _tile_tasks(e: int, start: int, count: int, tok_base: int, group: int, window: int, qt: int, row_tiles: int = 1):
+def _tile_tasks(e: int, start: int, count: int, tok_base: int, group: int, window: int, qt: int, row_tiles: int = 1,
+                keep: int = 0):
     """The tasks of an entry that is not split along its keys, without a loop over its tiles: (keys per group of
     four tasks, tasks [groups, 4, 12]).  A tile is ``qt`` tokens times ``group`` heads, cut into pieces of
     32 * ``row_tiles`` rows, a task each; pieces are padded to fours with empty tasks."""
@@ -254,9 +289,7 @@ def _tile_tasks(e: int, start: int, count: int, tok_base: int, group: int, windo
     fours = -(-pieces // 4)
     tok0 = np.arange(0, count, qt, dtype=np.int64)                           # [tiles]
     last = np.minimum(tok0 + qt, count)
-    k_end = start + last
-    lo = first_key(start + tok0, window)
-    kb = (lo // 32) * 32
+    kb, k_end = walk(start + tok0, start + last, window, keep)
     tiles = len(tok0)
     t = np.empty((tiles, fours * 4, 12), dtype=np.int32)
     t[:] = _NULL_TASK
@@ -307,7 +340,7 @@ def _serpentine(n: int, kv_heads: int, compute_units: int, head_size: int = 64) 
 
 def build_tasks(starts: np.ndarray, counts: np.ndarray, group: int, window: int, bucket_keys: Optional[int] = None,
                 vectorized: bool = True, *, kv_heads: int, max_waves: int = 2, row_tiles: int = 1,
-                head_size: int = 64, compute_units: int = 256) -> Tuple[np.ndarray, tuple]:
+                head_size: int = 64, compute_units: int = 256, keep: int = 0) -> Tuple[np.ndarray, tuple]:
     """Task records [n, 12] int32 (main tasks, then combine tasks), and (n_main, n_combine, n_partials, waves that
     share a task: two when a prompt tile walks many keys, else what ``chunk_for`` says for the split entries; pieces
     of 32 rows that a task which writes the output covers: ``row_tiles`` if the step has such tasks, walks at least
@@ -317,11 +350,13 @@ def build_tasks(starts: np.ndarray, counts: np.ndarray, group: int, window: int,
     Main tasks are padded to a multiple of 4 (one workgroup runs 4) and ordered so that tasks sharing keys are
     neighbours and long tasks come first.  With ``bucket_keys`` (decode steps: one token per entry; the context
     length that the step's graph serves, in tokens) every entry is split and owns the chunk slots of that many keys,
-    used or not, so all counts depend on (entries, bucket_keys) alone.
+    used or not, so all counts depend on (entries, bucket_keys) alone.  ``keep``: a request's first keys that its window
+    keeps (0 without a window): key ranges then count along the ``walk``.
     """
     bucket = bucket_keys
+    keep = keep if window > 0 else 0
     if vectorized and bucket is not None and len(counts) and int(counts.max()) == 1:
-        return _build_decode_tasks(starts, group, window, bucket, kv_heads, max_waves, head_size)
+        return _build_decode_tasks(starts, group, window, bucket, kv_heads, max_waves, head_size, keep)
     # two pieces of rows a task where the prompt tiles of the step walk long key ranges (see the kernel), and the
     # head size allows it
     longest = int((starts + counts).max()) if len(starts) else 0
@@ -337,15 +372,17 @@ def build_tasks(starts: np.ndarray, counts: np.ndarray, group: int, window: int,
 
     def splits(e):
         first = int(first_key(int(starts[e]), window))
-        return bucket is not None or (int(counts[e]) <= SPLIT_MAX_TOKENS
-                                      and int(starts[e]) + int(counts[e]) - first >= SPLIT_MIN_KEYS)
+        end = int(starts[e]) + int(counts[e])
+        if keep:
+            first, end = (int(v) for v in walk(int(starts[e]), end, window, keep))
+        return bucket is not None or (int(counts[e]) <= SPLIT_MAX_TOKENS and end - first >= SPLIT_MIN_KEYS)
 
     split_entries = [e for e in range(len(starts)) if splits(e)]
     chunk, waves, merge = CHUNK, 1, False
     if split_entries:
         most = bucket if bucket is not None else max(int(starts[e]) + int(counts[e]) for e in split_entries)
         if bucket is not None and window != 0:
-            most = min(most, abs(window) + CHUNK)
+            most = min(most, abs(window) + CHUNK + keep)
         chunk, waves = chunk_for(len(split_entries), most, kv_heads)
         waves = min(waves, max_waves)
         merge = merges_in_kernel(most)
@@ -356,20 +393,23 @@ def build_tasks(starts: np.ndarray, counts: np.ndarray, group: int, window: int,
         do_split = splits(e)
         tail = (int(tok_bases[e]), count, start, 0)
         if vectorized and not do_split:
-            lengths, groups = _tile_tasks(e, start, count, int(tok_bases[e]), group, window, qt, row_tiles)
+            lengths, groups = _tile_tasks(e, start, count, int(tok_bases[e]), group, window, qt, row_tiles,
+                                          keep)
             direct_arrays.append((lengths, groups))
             continue
         for tok0 in range(0, count, qt):
             last = min(tok0 + qt, count)
             k_end = start + last
             lo = int(first_key(start + tok0, window))
+            if keep:
+                lo, k_end = (int(v) for v in walk(start + tok0, k_end, window, keep))
             # pieces of the tile that hold at least one live row (the last tile of an entry may be short): 32 rows
             # each for tasks that leave partial results, 32 * row_tiles for those that write the output
             live = _live_pieces(rows, qt, min(qt, count - tok0), 32 if do_split else piece)
             if do_split:
                 c_first, c_last = lo // chunk, (k_end - 1) // chunk
                 # slot j holds chunk c_first + j
-                slots = _chunk_slots(bucket, chunk, window) if bucket is not None else c_last - c_first + 1
+                slots = _chunk_slots(bucket, chunk, window, keep) if bucket is not None else c_last - c_first + 1
                 for row0 in live:
                     piece_index = len(combine)       # a chunk's task names the record of its row piece
                     combine.append((e, tok0, qt, row0, 0, 0, n_part, c_last - c_first + 1) + tail)
@@ -416,15 +456,17 @@ def build_tasks(starts: np.ndarray, counts: np.ndarray, group: int, window: int,
 
 
 def _build_decode_tasks(starts: np.ndarray, group: int, window: int, bucket: int, kv_heads: int,
-                        max_waves: int = 2, head_size: int = 64):
+                        max_waves: int = 2, head_size: int = 64, keep: int = 0):
     """``build_tasks`` for a step in which every entry brings one token, without a Python loop over entries."""
     s = len(starts)
     starts = starts.astype(np.int64)
     k_end = starts + 1
     lo = first_key(starts, window)
+    if keep:
+        lo, k_end = walk(starts, k_end, window, keep)
     row_chunks = -(-group // 32)
     # the bucket, not the step's longest request, decides between whole ranges and chunks: a graph holds one of them
-    keys = bucket if window == 0 else min(bucket, abs(window) + CHUNK)      # what a token can see
+    keys = bucket if window == 0 else min(bucket, abs(window) + CHUNK + keep)      # what a token can see
     chunk, waves = chunk_for(s, keys, kv_heads, whole_ok=max_waves >= 8, head_size=head_size)
     waves = min(waves, max_waves)
     if chunk == 0:
@@ -439,7 +481,7 @@ def _build_decode_tasks(starts: np.ndarray, group: int, window: int, bucket: int
         whole[..., 9] = 1
         whole[..., 10] = starts[:, None]
         return whole.reshape(-1, 12), (s * row_chunks, 0, 0, waves, 1, False)
-    slots = _chunk_slots(bucket, chunk, window)
+    slots = _chunk_slots(bucket, chunk, window, keep)
     j = np.arange(slots, dtype=np.int64)
     c_first, c_last = lo // chunk, (k_end - 1) // chunk
     c = c_first[:, None] + j[None, :]                          # [s, slots]: slot j holds chunk c_first + j
@@ -478,8 +520,8 @@ def _build_decode_tasks(starts: np.ndarray, group: int, window: int, bucket: int
     return arr, (len(main), s * row_chunks, s * row_chunks * slots, waves, 1, merges_in_kernel(keys, waves))
 
 
-def plan_key(group: int, window: int, kv_heads: int, hd: int):
-    return ("attention_mfma_tasks", group, window, kv_heads, hd)
+def plan_key(group: int, window: int, kv_heads: int, hd: int, vd: Optional[int] = None, keep: int = 0):
+    return ("attention_mfma_tasks", group, window, kv_heads, hd, hd if vd is None else vd, keep)
 
 
 # Counters of the chunks that have finished, one per (row piece whose keys are cut into chunks, KV head): zeros that
@@ -500,44 +542,53 @@ def _merge_counters(device: torch.device, needed: int) -> Optional[torch.Tensor]
     return t
 
 
-def try_attention(q, k_cache, v_cache, out, ctx, cache, scale, window, nh, nkv, hd, sinks=None) -> bool:
-    """Run the fast kernels if they take this shape; False sends the caller to the general kernel."""
+def try_attention(q, k_cache, v_cache, out, ctx, cache, scale, window, nh, nkv, hd, sinks=None, *, vd=None, keep=0,
+                  slopes=None) -> bool:
+    """Run the fast kernels if they take this shape; False sends the caller to the general kernel.  ``vd``: columns of a
+    value head (default ``hd``); ``keep``: first keys that a window keeps; ``slopes``: float32 [nh], head h's score of
+    the key at j for the query at p gains slopes[h] * (j - p)."""
     page = cache.page_size
-    if not page_ok(page) or hd % 16 or not 16 <= hd <= 256:
+    vd = hd if vd is None else vd
+    keep = keep if window > 0 else 0
+    biased = bool(keep) or slopes is not None
+    if not page_ok(page) or hd % 16 or not 16 <= hd <= 256 or vd % 16 or not 16 <= vd <= 256:
         return False
+    if slopes is not None and not (slopes.dtype is torch.float32 and slopes.is_contiguous() and slopes.numel() == nh):
+        raise ValueError("slopes must be contiguous float32, one per query head")
     if sinks is not None and not (sinks.dtype is torch.float32 and sinks.is_contiguous() and sinks.numel() == nh):
         raise ValueError("sinks must be contiguous float32, one per query head")
     if q.stride(0) % 8 or q.data_ptr() % 16 or out.stride(0) % 4:
         return False
-    if tuple(k_cache.shape[1:]) != (nkv, page * hd) or tuple(v_cache.shape[1:]) != (nkv, page * hd):
+    if tuple(k_cache.shape[1:]) != (nkv, page * hd) or tuple(v_cache.shape[1:]) != (nkv, page * vd):
         raise ValueError("cache tensors must be [pages, nkv, page_size * hd] tiles")
     group = nh // nkv
-    plan = getattr(ctx, "plans", {}).get(plan_key(group, window, nkv, hd))
+    plan = getattr(ctx, "plans", {}).get(plan_key(group, window, nkv, hd, vd, keep))
     if plan is None:
         # a caller without a step planner (a kernel test): plan here and now
-        key = ("attention_tasks_adhoc", group, window, nkv, hd)
+        key = ("attention_tasks_adhoc", group, window, nkv, hd, vd, keep)
         plan = ctx.scratch.get(key)
         if plan is None:
             arr, meta = build_tasks(ctx.h_starts, ctx.h_counts, group, window, kv_heads=nkv,
-                                    max_waves=max_waves_for(hd), row_tiles=max_row_tiles_for(hd))
+                                    max_waves=max_waves_for(hd, vd), row_tiles=max_row_tiles_for(hd, vd), keep=keep)
             plan = (torch.from_numpy(arr).to(q.device), meta)
             ctx.scratch[key] = plan
     tasks, (n_main, n_comb, n_part, waves, row_tiles, merge) = plan
-    ksplit = min(waves, lib(hd, page=page).atoma_attention_mfma_max_ksplit())
+    module = lib(hd, page=page, vd=vd, biased=biased)
+    ksplit = min(waves, module.atoma_attention_mfma_max_ksplit())
     part_o = part_lse = None
     if n_part:
-        ws_key = ("attention_partials", nkv, hd)
+        ws_key = ("attention_partials", nkv, vd)
         ws = ctx.scratch.get(ws_key)
         if ws is None or ws[0].shape[0] < n_part:
-            ws = (torch.empty((n_part, nkv, 32, hd), dtype=torch.float32, device=q.device),
+            ws = (torch.empty((n_part, nkv, 32, vd), dtype=torch.float32, device=q.device),
                   torch.empty((n_part, nkv, 32), dtype=torch.float32, device=q.device))
             ctx.scratch[ws_key] = ws
         part_o, part_lse = ws
     bt = cache.block_tables
     counters = _merge_counters(q.device, n_comb * nkv) if n_comb and merge else None
-    _check(lib(hd, page=page).atoma_attention_mfma(_p(q), q.stride(0), _p(k_cache), _p(v_cache), _p(out), out.stride(0),
-                                        _p(part_o), _p(part_lse), _p(tasks), n_main, n_comb, _p(bt), bt.shape[1],
-                                        ctypes.c_float(scale), int(window), nh, nkv, ksplit, row_tiles, _p(counters),
-                                        _p(sinks), _stream()),
+    _check(module.atoma_attention_mfma(_p(q), q.stride(0), _p(k_cache), _p(v_cache), _p(out), out.stride(0),
+                                       _p(part_o), _p(part_lse), _p(tasks), n_main, n_comb, _p(bt), bt.shape[1],
+                                       ctypes.c_float(scale), int(window), nh, nkv, ksplit, row_tiles, _p(counters),
+                                       _p(sinks), int(keep), _p(slopes), _stream()),
            "attention_mfma")
     return True

@@ -9,7 +9,7 @@ from __future__ import annotations
 
 import ctypes
 import dataclasses
-from typing import Optional
+from typing import Optional, Tuple
 
 import torch
 
@@ -97,6 +97,26 @@ def embed(tokens: torch.Tensor, table: torch.Tensor, out: Optional[torch.Tensor]
     _need(out.dtype is torch.float32 and out.is_contiguous() and tuple(out.shape) == (n, width), "embed: bad out")
     _check(core().atoma_embed(_p(tokens), _p(table), _code(table, "embedding table"), _p(out), n, width,
                               table.shape[0], ctypes.c_float(scale), _stream()), "embed")
+    return out
+
+
+def embed_sinusoid(tokens: torch.Tensor, table: torch.Tensor, positions: torch.Tensor, freq: torch.Tensor,
+                   scale: float = 1.0, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """out[t, c] = table[tokens[t], c] * scale + (sin if c is even, else cos)(positions[t] * freq[c // 2]) as float32;
+    ``freq`` float64, one per pair of columns."""
+    _dev(tokens, table, positions, freq)
+    _i32(tokens, "tokens")
+    n, width = tokens.numel(), table.shape[1]
+    _i32(positions, "positions", n)
+    _need(table.dim() == 2 and table.is_contiguous(), "embedding table must be contiguous [vocab, width]")
+    _need(freq.dtype is torch.float64 and freq.is_contiguous() and freq.numel() == (width + 1) // 2,
+          "freq must be float64, one per pair of columns")
+    if out is None:
+        out = torch.empty((n, width), dtype=torch.float32, device=table.device)
+    _need(out.dtype is torch.float32 and out.is_contiguous() and tuple(out.shape) == (n, width), "embed: bad out")
+    _check(core().atoma_embed_sinusoid(_p(tokens), _p(table), _code(table, "embedding table"), _p(out), _p(positions),
+                                       _p(freq), n, width, table.shape[0], ctypes.c_float(scale), _stream()),
+           "embed_sinusoid")
     return out
 
 
@@ -206,22 +226,25 @@ def paged_attention_generic(q: torch.Tensor, kcache: torch.Tensor, vcache: torch
                             block_tables: torch.Tensor, token_seq: torch.Tensor, positions: torch.Tensor,
                             scale: float, window: int, page_size: int, nh: int, nkv: int, hd: int,
                             slopes: Optional[torch.Tensor] = None, chunk: int = 0,
-                            sinks: Optional[torch.Tensor] = None) -> None:
+                            sinks: Optional[torch.Tensor] = None, keep: int = 0, vd: Optional[int] = None) -> None:
     """Attention of every token of ``q`` [T, >= nh hd] (row stride free) over its request's cached keys.
 
     Token t belongs to row ``token_seq[t]`` of ``block_tables`` and sits at absolute position ``positions[t]``;
     it sees keys max(0, p - window + 1) .. p (window 0: all).  ``out`` is [T, nh hd].  ``slopes`` (float32 [nh]):
     head h's score of key j gains ``slopes[h] * (j - p)``.  ``chunk`` > 0: it sees only keys from (p // chunk) * chunk
-    on.  ``sinks`` (float32 [nh]): the softmax denominator also holds exp(sinks[h]).
+    on.  ``sinks`` (float32 [nh]): the softmax denominator also holds exp(sinks[h]).  ``keep``: it also sees the first
+    so many keys, wherever its window is.  ``vd``: columns of a value head (default ``hd``); ``out`` is then [T, nh vd].
     """
+    vd = hd if vd is None else int(vd)
+    _need(keep >= 0, "keep must not be negative")
     _dev(q, kcache, vcache, out, block_tables, token_seq, positions)
     t = q.shape[0]
     _need(q.dim() == 2 and q.stride(1) == 1 and q.shape[1] >= nh * hd, "q: bad shape")
-    _need(out.dim() == 2 and out.stride(1) == 1 and out.shape[0] == t and out.shape[1] >= nh * hd
+    _need(out.dim() == 2 and out.stride(1) == 1 and out.shape[0] == t and out.shape[1] >= nh * vd
           and out.dtype is q.dtype, "out: bad shape")
     pages = kcache.shape[0]
     _need(kcache.is_contiguous() and vcache.is_contiguous() and tuple(kcache.shape) == (pages, nkv, page_size * hd)
-          and tuple(vcache.shape) == (pages, nkv, page_size * hd) and kcache.dtype is vcache.dtype,
+          and tuple(vcache.shape) == (pages, nkv, page_size * vd) and kcache.dtype is vcache.dtype,
           "cache tensors must be [pages, nkv, page_size * hd] tiles")
     _need(block_tables.dim() == 2 and block_tables.dtype is torch.int32 and block_tables.is_contiguous(),
           "block_tables must be contiguous int32 [requests, blocks]")
@@ -239,7 +262,7 @@ def paged_attention_generic(q: torch.Tensor, kcache: torch.Tensor, vcache: torch
     _check(core().atoma_paged_attention_generic(
         _p(q), q.stride(0), _p(kcache), _p(vcache), _p(out), out.stride(0), _code(q, "q"), _code(kcache, "cache"),
         _p(block_tables), block_tables.shape[1], _p(token_seq), _p(positions), ctypes.c_float(scale), int(window),
-        page_size, t, nh, nkv, hd, _p(slopes), int(chunk), _p(sinks), _stream()), "paged_attention_generic")
+        page_size, t, nh, nkv, hd, _p(slopes), int(chunk), _p(sinks), int(keep), vd, _stream()), "paged_attention_generic")
 
 
 GATE_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1, "relu": 2, "clamped_sigmoid": 3}
@@ -318,7 +341,11 @@ def _f32(t: torch.Tensor, what: str, n: Optional[int] = None):
 
 
 def _term(delta: torch.Tensor, t: int, width: int):
-    """(pointer, dtype code, planes, plane stride) of a delta [T, W] or of planes [S, T, W]."""
+    """(pointer, dtype code, planes, plane stride) of a delta [T, W], of planes [S, T, W], or of one row [W] that joins
+    every row of the stream."""
+    if delta.dim() == 1:
+        _need(delta.is_contiguous() and delta.numel() == width, "a row of the stream's width is needed")
+        return _p(delta), _code(delta, "term"), 1, ctypes.c_size_t(0)
     _need(delta.is_contiguous() and tuple(delta.shape[-2:]) == (t, width) and delta.dim() in (2, 3),
           "a term must be contiguous [T, W] or [planes, T, W] and match resid")
     planes = delta.shape[0] if delta.dim() == 3 else 1
@@ -329,8 +356,8 @@ def add_normed(resid: torch.Tensor, terms, w_post: Optional[torch.Tensor], eps_p
                w_next: Optional[torch.Tensor] = None, eps_next: float = 0.0,
                out_dtype: Optional[torch.dtype] = None) -> Optional[torch.Tensor]:
     """resid += rmsnorm(sum_i scale_i * term_i) * w_post (float32, in place); with ``w_next`` also returns
-    rmsnorm(resid) * w_next in ``out_dtype``.  ``terms``: one or two (tensor, scale) pairs, each tensor [T, W] or
-    planes [S, T, W] (summed), float32 or bfloat16.  Norm weights are float32.  Without ``w_post`` the sum joins the
+    rmsnorm(resid) * w_next in ``out_dtype``.  ``terms``: one or two (tensor, scale) pairs, each tensor [T, W],
+    planes [S, T, W] (summed) or one row [W] for all, float32 or bfloat16.  Norm weights are float32.  Without ``w_post`` the sum joins the
     stream as it is: resid += sum_i scale_i * term_i."""
     _need(resid.dtype is torch.float32 and resid.dim() == 2 and resid.is_contiguous(), "resid must be float32 [T, W]")
     t, width = resid.shape
@@ -674,15 +701,41 @@ def head_linear(x: torch.Tensor, w: torch.Tensor, out_dtype: torch.dtype, gate: 
 
 
 
+def head_norm(proj: torch.Tensor, wq: torch.Tensor, wk: torch.Tensor, eps: float, kcache: torch.Tensor,
+              vcache: torch.Tensor, slot_mapping: torch.Tensor, page_size: int, nh: int, nkv: int, hd: int, vd: int,
+              hd_out: int, vd_out: int, out_dtype: torch.dtype) -> torch.Tensor:
+    """From proj float32 [T, >= nh hd + nkv hd + nkv vd] (q, k, v): every q and k head divided by its root mean square
+    and multiplied by ``wq`` / ``wk`` [hd]; returns q [T, nh hd_out] and writes k and v into the tiles at
+    ``slot_mapping``.  Columns beyond ``hd`` / ``vd`` are zeros."""
+    _dev(proj, wq, wk, kcache, vcache, slot_mapping)
+    t = proj.shape[0]
+    _need(proj.dtype is torch.float32 and proj.dim() == 2 and proj.stride(1) == 1
+          and proj.shape[1] >= (nh + nkv) * hd + nkv * vd, "head_norm: proj must be float32 [T, >= q, k and v columns]")
+    _f32(wq, "q norm weight", hd)
+    _f32(wk, "k norm weight", hd)
+    _i32(slot_mapping, "slot_mapping", t)
+    pages = kcache.shape[0]
+    _need(kcache.is_contiguous() and vcache.is_contiguous() and kcache.dtype is out_dtype and vcache.dtype is out_dtype
+          and tuple(kcache.shape) == (pages, nkv, page_size * hd_out)
+          and tuple(vcache.shape) == (pages, nkv, page_size * vd_out), "head_norm: bad tiles")
+    q = torch.empty((t, nh * hd_out), dtype=out_dtype, device=proj.device)
+    _check(_module("layer_norms").atoma_head_norm(
+        _p(proj), proj.stride(0), _p(slot_mapping), _p(wq), _p(wk), ctypes.c_float(eps), _p(q), _p(kcache), _p(vcache),
+        _code(q, "q"), int(page_size), t, nh, nkv, hd, vd, hd_out, vd_out, _stream()), "head_norm")
+    return q
+
+
 ROUTER_SCORES = {"sigmoid": 0, "softmax": 1, "softmax_chosen": 2}
 
 
 def route_topk(logits: torch.Tensor, top: int, score: str = "sigmoid", correction: Optional[torch.Tensor] = None,
-               scale: float = 1.0, bias: Optional[torch.Tensor] = None):
+               scale: float = 1.0, bias: Optional[torch.Tensor] = None, groups: Optional[Tuple[int, int]] = None):
     """(ids int32 [T, top], weights float32 [T, top]).  Scores are sigmoid(logits) or ("softmax") the softmax of a
     row; the ``top`` experts with the largest score + ``correction`` [experts] are chosen and weighed by
     score * ``scale``.  "softmax_chosen": the largest logits are chosen and weighed by the softmax over the chosen
-    ones, times ``scale``.  ``bias`` [experts] joins the logits first."""
+    ones, times ``scale``.  ``bias`` [experts] joins the logits first.  ``groups`` = (count, keep): the experts form
+    ``count`` equal runs of neighbours, a run's score is its best expert's, and only experts of the best ``keep`` runs
+    can be chosen."""
     _dev(logits, correction, bias)
     _need(score in ROUTER_SCORES, f"route_topk: scores are one of {', '.join(ROUTER_SCORES)}")
     _need(score != "softmax_chosen" or correction is None, "route_topk: a correction needs scores of its own")
@@ -696,7 +749,8 @@ def route_topk(logits: torch.Tensor, top: int, score: str = "sigmoid", correctio
     scores = torch.empty((t, top), dtype=torch.float32, device=logits.device)
     _check(_module("experts").atoma_route_topk(_p(logits), logits.stride(0), e, int(top), _p(ids), _p(scores), t,
                                                ROUTER_SCORES[score], _p(correction), ctypes.c_float(scale), _p(bias),
-                                               _stream()), "route_topk")
+                                               *((int(g) for g in groups) if groups else (0, 0)), _stream()),
+           "route_topk")
     return ids, scores
 
 

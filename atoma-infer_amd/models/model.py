@@ -47,23 +47,25 @@ class Model:
         readers = [b.entry_norm() for b in blocks[1:]]
         readers.append(spec.final_norm[1] if getattr(ctx, "wants_all_rows", False) else None)
         first = blocks[0].entry_norm() if blocks else None
+        # (an embedding that adds something of the tokens' positions is handed them)
+        where = {"positions": ctx.positions} if getattr(spec.embedding[1], "reads_positions", False) else {}
         if getattr(spec.embedding[1], "reads_context", False):
             # an embedding that reads more of the step than its tokens (positions, entries, a state of its own)
             from ..cache.pool import EMBEDDING_CALL
             resid, pending = spec.embedding[1].forward_step(ctx, ctx.layer_cache(EMBEDDING_CALL)), None
         elif first is not None:
-            resid, pending = spec.embedding[1].forward(ctx.tokens, first)
+            resid, pending = spec.embedding[1].forward(ctx.tokens, first, **where)
         else:
-            resid, pending = spec.embedding[1].forward(ctx.tokens), None
+            resid, pending = spec.embedding[1].forward(ctx.tokens, **where), None
         # a block that maps the stream from the embedding's rows too gets them as they were (gathered once more: the
         # stream's own rows are summed into in place), and one that is run several times is told which run this is
-        embedded = spec.embedding[1].forward(ctx.tokens) if any(getattr(b, "reads_embedding", False) for b in blocks) \
+        embedded = spec.embedding[1].forward(ctx.tokens, **where) if any(getattr(b, "reads_embedding", False) for b in blocks) \
             else None
         # blocks that weigh the results of all blocks before them: the results of one step, the embedding's rows first
         results = None
         if any(getattr(b, "keeps_results", False) for b in blocks):
             results = torch.empty((len(blocks) + 1, *resid.shape), dtype=torch.float32, device=resid.device)
-            spec.embedding[1].forward(ctx.tokens, out=results[0])
+            spec.embedding[1].forward(ctx.tokens, out=results[0], **where)
         runs = {}
         for pos, block in enumerate(blocks):
             extra = {}

@@ -31,6 +31,7 @@ class PagedAttention(Mixer):
     def __init__(self, width: int, num_heads: int, num_kv_heads: int, head_size: int,
                  position: Optional[PositionEncoding] = None, window: Optional[int] = None,
                  scale: Optional[float] = None, chunk: Optional[int] = None, value_size: Optional[int] = None,
+                 keep_first: int = 0,
                  names=("q_proj.weight", "k_proj.weight", "v_proj.weight", "o_proj.weight")):
         if num_heads % num_kv_heads:
             raise ValueError(f"{num_heads} query heads cannot be grouped over {num_kv_heads} KV heads")
@@ -49,9 +50,15 @@ class PagedAttention(Mixer):
             raise ValueError("window must be positive")
         if chunk is not None and (chunk <= 0 or window is not None):
             raise ValueError("chunk must be positive, and a layer has a window or chunks, not both")
+        if keep_first < 0:
+            raise ValueError("keep_first must not be negative")
         self.width, self.nh, self.nkv, self.hd = int(width), int(num_heads), int(num_kv_heads), int(head_size)
         self.position = position
         self.window = window
+        # keep_first k: beside its window a token sees the keys 0 .. k - 1 of its request (without a window it sees all)
+        self.keep_first = int(keep_first) if window is not None else 0
+        # columns of a cached value head (a subclass may cache values of another width than its keys)
+        self.value_hd = self.hd
         # chunk c: the token at p sees keys (p // c) * c .. p only, chunks counted from the request's first position
         self.chunk = chunk
         self.sinks: Optional[torch.Tensor] = None       # float32 [heads]: exp(sinks[h]) joins the softmax denominator
@@ -83,21 +90,25 @@ class PagedAttention(Mixer):
         return torch.nn.functional.pad(w.view(w.shape[0], heads, size), (0, to - size)).reshape(w.shape[0], heads * to)
 
     def cache_spec(self) -> CacheSpec:
-        return CacheSpec(self.nkv, self.hd, self.window, chunk=self.chunk)
+        return CacheSpec(self.nkv, self.hd, self.window, chunk=self.chunk, keep_first=self.keep_first,
+                         value_size=None if self.value_hd == self.hd else self.value_hd)
+
+    def _load_position(self, get, device, act_dtype) -> None:
+        if self.position is not None:
+            self.position.load(get, device, act_dtype)
+        self.slopes = self.position.score_slopes(self.nh) if self.position is not None else None
+        if self.slopes is not None:
+            self.slopes = self.slopes.to(device=device, dtype=torch.float32).contiguous()
+            if self.slopes.numel() != self.nh:
+                raise ValueError(f"score_slopes gave {self.slopes.numel()} slopes for {self.nh} heads")
 
     def load(self, get, device, act_dtype) -> None:
         ws = [self._pad_heads(get(self.names[0]), self.nh, self.hd_in, self.hd, True),
               self._pad_heads(get(self.names[1]), self.nkv, self.hd_in, self.hd, True),
               self._pad_heads(get(self.names[2]), self.nkv, self.vd_in, self.hd, True)]
         dt = ws[0].dtype if all(w.dtype is ws[0].dtype for w in ws) else torch.float32
-        if self.position is not None:
-            self.position.load(get, device, act_dtype)
+        self._load_position(get, device, act_dtype)
         tables = self.position.rotary_tables() if self.position is not None else None
-        self.slopes = self.position.score_slopes(self.nh) if self.position is not None else None
-        if self.slopes is not None:
-            self.slopes = self.slopes.to(device=device, dtype=torch.float32).contiguous()
-            if self.slopes.numel() != self.nh:
-                raise ValueError(f"score_slopes gave {self.slopes.numel()} slopes for {self.nh} heads")
         self.paired = tables is not None and tables[2] == self.hd
         if self.paired:
             half = self.hd // 2
@@ -123,8 +134,6 @@ class PagedAttention(Mixer):
         kernels, built once per step on the host and shipped with the step's metadata.  ``bucket_tokens`` is None, or
         for a step that only decodes the context length its plan must serve (a multiple of the runner's bucket)."""
         from ..kernels import attention_bf16
-        if self.slopes is not None:
-            return None          # scores with a bias take the general kernel, which needs no plan
         if cache_dtype is torch.bfloat16 and self.hd % 16:
             import warnings
             warnings.warn(f"bfloat16 attention with heads of {self.hd} columns runs the general kernel (one wave per "
@@ -138,13 +147,14 @@ class PagedAttention(Mixer):
                           f"multiple of 16 tokens ([cache] block_size = 16, 32, 64, ...)", stacklevel=2)
         if cache_dtype is not torch.bfloat16 or not attention_bf16.page_ok(page_size):
             return None
-        group, window, nkv = self.nh // self.nkv, self.span, self.nkv
+        group, window, nkv, vd, keep = self.nh // self.nkv, self.span, self.nkv, self.value_hd, self.keep_first
         cus = torch.cuda.get_device_properties(self.w_o.device).multi_processor_count
-        return (attention_bf16.plan_key(group, window, nkv, self.hd),
+        return (attention_bf16.plan_key(group, window, nkv, self.hd, vd, keep),
                 lambda starts, counts, bucket: attention_bf16.build_tasks(
                     starts, counts, group, window, bucket, kv_heads=nkv,
-                    max_waves=attention_bf16.max_waves_for(self.hd),
-                    row_tiles=attention_bf16.max_row_tiles_for(self.hd), head_size=self.hd, compute_units=cus))
+                    max_waves=attention_bf16.max_waves_for(self.hd, vd),
+                    row_tiles=attention_bf16.max_row_tiles_for(self.hd, vd), head_size=self.hd, compute_units=cus,
+                    keep=keep))
 
     @property
     def span(self) -> int:
@@ -200,14 +210,15 @@ class PagedAttention(Mixer):
         return linear_delta(out, self.w_o, sink, self.w_o_tiled)
 
     def attend(self, q, k_cache, v_cache, out, ctx, cache) -> None:
-        if self.slopes is None and q.dtype is torch.bfloat16 and k_cache.dtype is torch.bfloat16:
+        if q.dtype is torch.bfloat16 and k_cache.dtype is torch.bfloat16:
             from ..kernels import attention_bf16
             if attention_bf16.try_attention(q, k_cache, v_cache, out, ctx, cache, self.scale, self.span,
-                                            self.nh, self.nkv, self.hd, self.sinks):
+                                            self.nh, self.nkv, self.hd, self.sinks, vd=self.value_hd,
+                                            keep=self.keep_first, slopes=self.slopes):
                 return
         ops.paged_attention_generic(q, k_cache, v_cache, out, cache.block_tables, ctx.token_seq, ctx.positions,
                                     self.scale, self.window or 0, cache.page_size, self.nh, self.nkv, self.hd,
-                                    self.slopes, self.chunk or 0, self.sinks)
+                                    self.slopes, self.chunk or 0, self.sinks, self.keep_first, self.value_hd)
 
 
 class TiedValueAttention(PagedAttention):
@@ -292,6 +303,83 @@ class TiedValueAttention(PagedAttention):
         out = torch.empty((t, nh * hd), dtype=x.dtype, device=x.device)
         self.attend(q, cache.k, cache.v, out, ctx, cache)
         return linear_delta(out, self.w_o, None, self.w_o_tiled)
+
+
+class HeadNormAttention(PagedAttention):
+    """Attention whose queries and keys are normed head by head, without biases:
+
+    * every head of q and k is divided by its root mean square and multiplied by a plain weight of ``head_size`` numbers
+      that all heads share (``q.norm``, ``k.norm``); values have ``value_size`` columns and stay as projected;
+    * positions enter through ``position``, where it biases the scores by distance (``score_slopes``), and through the
+      mask: an optional window, beside which a token may see its request's first ``keep_first`` keys;
+    * with ``sink`` one learned number per head joins the softmax denominator (tensor ``sink``).
+
+    Keys and values are cached with their own widths, each rounded up to a multiple of 16 (zero columns).
+
+    Tensors ([out, in]): ``q``, ``k``, ``v``, ``o``, ``q.norm``, ``k.norm`` [head_size], ``sink`` [heads].
+    """
+
+    def __init__(self, width: int, num_heads: int, num_kv_heads: int, head_size: int, value_size: int, scale: float,
+                 norm_eps: float, position: Optional[PositionEncoding] = None, window: Optional[int] = None,
+                 keep_first: int = 0, sink: bool = True):
+        padded = -(-int(head_size) // 16) * 16
+        super().__init__(width, num_heads, num_kv_heads, padded, position, window, scale, None, keep_first=keep_first)
+        if not 0 < value_size <= 256:
+            raise ValueError("values of more than 256 columns a head are not supported")
+        if position is not None and position.rotary_tables() is not None:
+            raise ValueError("a rotation of normed heads is not supported")
+        self.hd_in, self.vd_in = int(head_size), int(value_size)
+        self.value_hd = -(-self.vd_in // 16) * 16
+        self.norm_eps, self.has_sink = float(norm_eps), bool(sink)
+        self.w_in = self.w_in_tiled = self.q_norm = self.k_norm = None
+
+    def weight_specs(self) -> Dict[str, WeightSpec]:
+        h, g, d, v, w = self.nh, self.nkv, self.hd_in, self.vd_in, self.width
+        specs = {"q": WeightSpec((h * d, w)), "k": WeightSpec((g * d, w)), "v": WeightSpec((g * v, w)),
+                 "o": WeightSpec((w, h * v)), "q.norm": WeightSpec((d,), "norm"), "k.norm": WeightSpec((d,), "norm")}
+        if self.has_sink:
+            specs["sink"] = WeightSpec((h,), "linear", std=1.0)
+        return specs
+
+    def load(self, get, device, act_dtype) -> None:
+        self._load_position(get, device, act_dtype)
+        ws = [get("q"), get("k"), get("v")]
+        dt = ws[0].dtype if all(w.dtype is ws[0].dtype for w in ws) else torch.float32
+        rows = sum(w.shape[0] for w in ws)
+        parts = [w.to(device=device, dtype=dt) for w in ws]
+        if (-rows) % 64:      # whole tiles for the matrix-core products
+            parts.append(torch.zeros(((-rows) % 64, self.width), dtype=dt, device=device))
+        self.w_in = torch.cat(parts, dim=0).contiguous()
+        self.w_o = self._pad_heads(get("o").to(device), self.nh, self.vd_in, self.value_hd, False).contiguous()
+        f32 = dict(device=device, dtype=torch.float32)
+        self.q_norm, self.k_norm = get("q.norm").to(**f32).contiguous(), get("k.norm").to(**f32).contiguous()
+        self.sinks = get("sink").to(**f32).contiguous() if self.has_sink else None
+        self.act_dtype = act_dtype
+        self.w_in_tiled = self.w_o_tiled = None
+        if act_dtype is torch.bfloat16 and self.w_in.dtype is torch.bfloat16 and self.w_o.dtype is torch.bfloat16:
+            from ..kernels import gemm_bf16
+            plan = gemm_bf16.tiled_plan(self.w_in.shape[0], self.width, swiglu=False)
+            if plan is not None:
+                self.w_in_tiled = gemm_bf16.tile_weight(self.w_in, *plan)
+            self.w_o_tiled = gemm_bf16.tile_copies_resid(self.w_o)
+
+    def device_bytes(self) -> int:
+        return sum(w.numel() * w.element_size() for w in (self.w_in, self.w_o))
+
+    accepts_begun = True
+    takes_sink = True
+
+    def forward(self, x, ctx, cache, sink=None):
+        if not cache.writable:
+            raise NotImplementedError("attention with normed heads reads only a cache of its own")
+        t = x.shape[0]
+        # the projections leave in float32: the norms are float32 work
+        proj = linear(x, self.w_in, torch.float32, tiled=self.w_in_tiled)
+        q = ops.head_norm(proj, self.q_norm, self.k_norm, self.norm_eps, cache.k, cache.v, cache.slot_mapping,
+                          cache.page_size, self.nh, self.nkv, self.hd_in, self.vd_in, self.hd, self.value_hd, x.dtype)
+        out = torch.empty((t, self.nh * self.value_hd), dtype=x.dtype, device=q.device)
+        self.attend(q, cache.k, cache.v, out, ctx, cache)
+        return linear_delta(out, self.w_o, sink, self.w_o_tiled)
 
 
 class LatentAttention(PagedAttention):
@@ -688,6 +776,7 @@ class RotaryLatentAttention(PagedAttention):
 register_mixer("latent_attention", LatentAttention)
 register_mixer("differential_attention", DifferentialAttention)
 register_mixer("attention", PagedAttention)
+register_mixer("head_norm_attention", HeadNormAttention)
 register_mixer("tied_value_attention", TiedValueAttention)
 register_mixer("gated_tied_value_attention", GatedTiedValueAttention)
 register_mixer("rotary_latent_attention", RotaryLatentAttention)

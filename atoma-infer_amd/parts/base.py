@@ -57,7 +57,8 @@ class WeightSpec:
 class CacheSpec:
     """What a mixer keeps per token: keys and values of ``kv_heads`` heads of ``head_size``.
 
-    ``window``: None keeps every token; w keeps the last w.  ``chunk``: c keeps the tokens of the current chunk of c
+    ``window``: None keeps every token; w keeps the last w, and with ``keep_first`` a request's first so many tokens
+    beside them (a window never loses those).  ``chunk``: c keeps the tokens of the current chunk of c
     positions (chunks count from the request's first position), for mixers whose tokens see their own chunk only.
     Layers whose specs are equal share one group of pages and one block table per request.
 
@@ -71,10 +72,11 @@ class CacheSpec:
     window: Optional[int] = None
     value_size: Optional[int] = None
     chunk: Optional[int] = None
+    keep_first: int = 0
 
     def __post_init__(self):
         if self.kv_heads <= 0 or self.head_size <= 0 or (self.value_size is not None and self.value_size < 0) \
-                or (self.window and self.chunk):
+                or (self.window and self.chunk) or self.keep_first < 0 or (self.keep_first and not self.window):
             raise ValueError(f"invalid cache spec: {self}")
 
     @property
@@ -199,9 +201,8 @@ class PositionEncoding(Part):
         raise NotImplementedError
 
     def score_slopes(self, num_heads: int) -> Optional[torch.Tensor]:
-        """float32 [num_heads] on the device, or None: an encoding that biases the attention scores by the distance,
-        head h's score of the key at j for the query at p gaining ``slopes[h] * (j - p)``.  Attention with such a
-        bias runs the general kernel (the matrix-core kernel has no bias)."""
+        """float32 [num_heads], or None: an encoding that biases the attention scores by the distance, head h's
+        score of the key at j for the query at p gaining ``slopes[h] * (j - p)``."""
         return None
 
 
@@ -241,7 +242,7 @@ class Block(Part):
     #: True if ``forward`` has a keyword ``next_norm``: the norm that will read this block's output (the next
     #: block's ``entry_norm()``, or the final norm), so that the block's last product may begin it
     fuses_next_norm = False
-    #: True if ``forward`` has a keyword ``embedded``: the float32 rows as the embedding left them
+    #: True if ``forward`` has a keyword ``embedded``: the float32 rows as the embedding left them (not to be changed)
     reads_embedding = False
     #: True if ``forward`` has keywords ``results`` and ``position``: a float32 tensor [blocks + 1, T, width] that lives
     #: for one step, whose row 0 holds the embedding's rows and row j + 1 is the block at run-order position j's to

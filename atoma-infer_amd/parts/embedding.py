@@ -16,8 +16,14 @@ from .linear import linear
 
 
 class TokenEmbedding(Part):
-    def __init__(self, vocab_size: int, width: int, name: str = "weight", scale: float = 1.0):
+    def __init__(self, vocab_size: int, width: int, name: str = "weight", scale: float = 1.0,
+                 sinusoid_base: Optional[float] = None):
         # ``scale`` multiplies the rows on their way into the stream; a head tied to the table reads it without
+        # ``sinusoid_base`` b: a vector of the token's position p is added to its row, sin(p b^(-2i / width)) in column
+        # 2i and the cosine of the same in column 2i + 1
+        self.sinusoid_base = None if sinusoid_base is None else float(sinusoid_base)
+        self.reads_positions = self.sinusoid_base is not None
+        self.freq: Optional[torch.Tensor] = None
         self.vocab_size, self.width, self.name, self.scale = int(vocab_size), int(width), str(name), float(scale)
         self.weight: Optional[torch.Tensor] = None
 
@@ -29,13 +35,19 @@ class TokenEmbedding(Part):
 
     def load(self, get, device, act_dtype) -> None:
         self.weight = get(self.name).to(device).contiguous()
+        if self.reads_positions:
+            i = torch.arange((self.width + 1) // 2, dtype=torch.float64)
+            self.freq = torch.pow(torch.tensor(self.sinusoid_base, dtype=torch.float64), -2.0 * i / self.width).to(device)
 
     def device_bytes(self) -> int:
         return 0  # a step reads only the rows of its tokens
 
-    def forward(self, tokens: torch.Tensor, norm=None, out=None):
+    def forward(self, tokens: torch.Tensor, norm=None, out=None, positions=None):
         """The float32 residual rows of ``tokens`` (into ``out`` where given); with ``norm`` (the norm that reads them
-        first) a pair (rows, that norm begun or None)."""
+        first) a pair (rows, that norm begun or None).  ``positions`` [T] is given where ``reads_positions`` says so."""
+        if self.reads_positions:
+            rows = ops.embed_sinusoid(tokens, self.weight, positions, self.freq, self.scale, out)
+            return rows if norm is None else (rows, None)
         if norm is None:
             return ops.embed(tokens, self.weight, out, self.scale)
         # (a norm that cannot begin scaled rows is not asked to)

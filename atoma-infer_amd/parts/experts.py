@@ -3,8 +3,9 @@
 ``RoutedExperts``: router logits ``z = W_r x`` (with ``router_bias``: ``+ b``) in float32; scores ``s = sigmoid(z)`` or ``softmax(z)`` over all
 experts; the ``top`` experts with the largest ``s + correction`` are chosen (``correction``: a tensor of one number
 an expert that only chooses; none: the scores alone; the lower index wins a tie) and weighed by ``s * scale`` as
-they are, without renormalising; or, with scores "softmax_chosen", the experts with the largest ``z`` are chosen and
-weighed by the softmax over the chosen ``z`` alone, times ``scale``.  Two forms of expert, no biases:
+they are, without renormalising; with ``groups`` = (count, keep) only experts of the ``keep`` best of ``count`` equal
+runs of neighbours (a run is as good as its best expert) can be chosen; or, with scores "softmax_chosen", the experts
+with the largest ``z`` are chosen and weighed by the softmax over the chosen ``z`` alone, times ``scale``.  Two forms of expert, no biases:
 
 * ``swiglu``: ``W_down act(W_gate z, W_up z)``, act by default silu(gate) * up (``activation``, as
   ``kernels.ops.gate_activation`` takes it); the weight multiplies the expert's *input*,
@@ -43,7 +44,8 @@ from .linear import linear, linear_delta
 class RoutedExperts(FeedForward):
     def __init__(self, width: int, intermediate: int, experts: int, top: int, score: str = "sigmoid",
                  scale: float = 1.0, correction: bool = False, expert: str = "swiglu", shared: int = 0,
-                 activation="silu", weigh: str = "input", router_bias: bool = False, shared_activation=None):
+                 activation="silu", weigh: str = "input", router_bias: bool = False, shared_activation=None,
+                 groups=None):
         if not 0 < top <= experts or experts > 1024:
             raise ValueError(f"{top} of {experts} experts: top must be at least 1 and at most the number of experts "
                              f"(up to 1,024)")
@@ -53,6 +55,12 @@ class RoutedExperts(FeedForward):
             raise ValueError("a weight multiplies an expert's 'input' or its 'output'")
         if correction and score == "softmax_chosen":
             raise ValueError("a correction chooses by scores, which 'softmax_chosen' does not have")
+        self.groups = None if groups is None else (int(groups[0]), int(groups[1]))
+        if groups is not None:
+            count, keep = self.groups
+            if count <= 0 or experts % count or not 0 < keep <= count or keep * (experts // count) < top:
+                raise ValueError(f"{experts} experts in {count} groups of which {keep} are kept: the groups must be equal "
+                                 f"and the kept ones hold the {top} chosen experts")
         ops.gate_activation(activation)
         self.width, self.inter, self.experts, self.top = int(width), int(intermediate), int(experts), int(top)
         self.score, self.scale, self.has_correction = str(score), float(scale), bool(correction)
@@ -168,7 +176,7 @@ class RoutedExperts(FeedForward):
 
     def forward(self, x, ctx):
         ids, weights = ops.route_topk(linear(x, self.w_router, torch.float32), self.top, self.score, self.correction,
-                                      self.scale, self.router_b)
+                                      self.scale, self.router_b, self.groups)
         out = self._routed(x, ids, weights)
         if not self.shared:
             return out

@@ -1,6 +1,6 @@
 """The entry of a pass over layers that run several times in a row with the same weights.
 
-Before the first layer of every pass the stream is mapped anew from itself and from the embedding's rows,
+``LoopEntry``: before the first layer of every pass the stream is mapped anew from itself and from the embedding's rows,
 
     x <- W_in [x; x0] + step[t],
 
@@ -9,6 +9,9 @@ order (it mixes nothing between tokens and keeps no cache), run once per pass; w
 it (``takes_turn``).  The product may run in the activation dtype; its sums, the bias and the new stream are float32.
 
 Tensors: ``in`` [width, 2 width] (the stream's columns first), ``step`` [times, width].
+
+``LoopStep``: the same without a map, ``x <- x + x0 + step[t]``, x0 joining before every pass but the first (or before
+all).  One kernel adds and norms what the pass's first layer reads.  Tensor: ``step`` [times, width].
 """
 from __future__ import annotations
 
@@ -74,5 +77,43 @@ class LoopEntry(Block):
         return None
 
 
+class LoopStep(Block):
+    reads_embedding = True
+    takes_turn = True
+    fuses_next_norm = True
+
+    def __init__(self, width: int, times: int, name: str = "step", embedding_from: int = 1):
+        """``embedding_from``: the first pass that the embedding's rows join (``times`` or more: none)."""
+        self.width, self.times, self.name, self.embedding_from = int(width), int(times), str(name), int(embedding_from)
+        self.reads_embedding = self.embedding_from < self.times
+        self.mixer = NoMixer()
+        self.steps: Optional[torch.Tensor] = None
+
+    def graph_safe(self) -> bool:
+        return True
+
+    def weight_specs(self) -> Dict[str, WeightSpec]:
+        return {self.name: WeightSpec((self.times, self.width), std=0.3)}
+
+    def load(self, get, device, act_dtype) -> None:
+        self.steps = get(self.name).to(device=device, dtype=torch.float32).contiguous()
+
+    def forward(self, resid, delta, ctx, cache, embedded=None, turn=0, next_norm=None):
+        if not 0 <= turn < self.times or (embedded is None and self.embedding_from <= turn):
+            raise RuntimeError("a loop step needs a pass number below its number of passes and the embedding's rows")
+        if isinstance(delta, (Begun, Normed)):
+            pass                        # the block before has added its outputs to the stream already
+        elif delta is not None:
+            ops.add_normed(resid, delta.terms if isinstance(delta, WeightedSum) else [(delta, 1.0)], None, 0.0)
+        terms = ([(embedded, 1.0)] if turn >= self.embedding_from else []) + [(self.steps[turn], 1.0)]
+        # (a norm that can only begin or only add finishes on its own)
+        if getattr(next_norm, "weight_f32", None) is None:
+            ops.add_normed(resid, terms, None, 0.0)
+            return None
+        return Normed(ops.add_normed(resid, terms, None, 0.0, next_norm.weight_f32, next_norm.eps, next_norm.act_dtype),
+                      next_norm)
+
+
 register_mixer("none", NoMixer)
 register_block("loop_entry", LoopEntry)
+register_block("loop_step", LoopStep)

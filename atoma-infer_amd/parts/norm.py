@@ -14,11 +14,15 @@ from .base import Begun, Norm, WeightedSum, WeightSpec, register_norm
 
 
 class RMSNorm(Norm):
-    def __init__(self, width: int, eps: float, name: str = "weight", offset: float = 0.0, scalar: bool = False):
+    def __init__(self, width: int, eps: float, name: str = "weight", offset: float = 0.0, scalar: bool = False,
+                 gain: Optional[str] = None, factor: float = 1.0):
         # ``name``: the tensor's name below the part's prefix ("weight" as checkpoints of the Llama family have it)
         # ``offset``: what is added to the stored tensor to make the weight (1 for weights stored around zero); such
         # a weight is kept in float32, since 1 + w has more digits than the checkpoint's dtype
         # ``scalar``: the checkpoint holds one number for all columns (a tensor without dimensions, or of one entry)
+        # ``gain``: a second tensor that multiplies the norm's result column by column, and ``factor`` a number for all
+        # columns (a layer scale and a residual multiplier behind a sublayer's norm): both become part of the weight
+        self.gain, self.factor = gain, float(factor)
         self.width, self.eps, self.name, self.offset = int(width), float(eps), str(name), float(offset)
         self.scalar = bool(scalar)
         self.weight: Optional[torch.Tensor] = None
@@ -29,7 +33,10 @@ class RMSNorm(Norm):
         return True
 
     def weight_specs(self) -> Dict[str, WeightSpec]:
-        return {self.name: WeightSpec(() if self.scalar else (self.width,), "norm" if self.offset == 0.0 else "norm_zero")}
+        specs = {self.name: WeightSpec(() if self.scalar else (self.width,), "norm" if self.offset == 0.0 else "norm_zero")}
+        if self.gain is not None:
+            specs[self.gain] = WeightSpec((self.width,), mean=0.7, std=0.1)
+        return specs
 
     def load(self, get, device, act_dtype) -> None:
         self.weight = get(self.name).to(device).contiguous()
@@ -37,6 +44,9 @@ class RMSNorm(Norm):
             self.weight = self.weight.reshape(1).expand(self.width).contiguous()
         if self.offset != 0.0:
             self.weight = (self.weight.to(torch.float32) + self.offset).contiguous()
+        if self.gain is not None or self.factor != 1.0:
+            gain = get(self.gain).to(device=device, dtype=torch.float32) if self.gain is not None else 1.0
+            self.weight = (self.weight.to(torch.float32) * gain * self.factor).contiguous()
         self.weight_f32 = self.weight.to(torch.float32)
         self.act_dtype = act_dtype
 

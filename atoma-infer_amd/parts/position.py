@@ -4,7 +4,8 @@
 frequencies are ``theta^(-2i/hd)`` (models/src/llama.rs:146-152), optionally rescaled by the llama3 rule
 (models/src/llama.rs:163-186).  The table of cos and sin is built once, in float32, for every position below
 ``max_positions`` (models/src/llama.rs:189-199) and stays float32 whatever the activation dtype is; all layers
-with equal parameters share it.  ``NoPosition`` encodes nothing.
+with equal parameters share it.  ``NoPosition`` encodes nothing.  ``DistanceBias`` rotates nothing and takes a multiple of
+the distance off the scores.
 """
 from __future__ import annotations
 
@@ -94,6 +95,18 @@ class NoPosition(PositionEncoding):
         return None
 
 
+class DistanceBias(NoPosition):
+    """The score of the key at j for the query at p loses ``slope_h (p - j)``, slope_h = 2^(-exponent (h + 1) / heads)
+    for head h = 0 .. heads - 1."""
+
+    def __init__(self, exponent: float = 8.0):
+        self.exponent = float(exponent)
+
+    def score_slopes(self, num_heads: int) -> torch.Tensor:
+        h = torch.arange(1, num_heads + 1, dtype=torch.float64)
+        return torch.pow(2.0, -self.exponent * h / num_heads).to(torch.float32)
+
+
 def clear_tables() -> None:
     _TABLES.clear()
 
@@ -123,3 +136,4 @@ def rotation_frequencies(base: float, dims: int, scaling: Optional[dict] = None)
 
 register_position("rotary", RotaryEncoding)
 register_position("none", NoPosition)
+register_position("distance_bias", DistanceBias)
