@@ -201,8 +201,10 @@ __device__ __forceinline__ void merge_parts(const float* __restrict__ part_o, co
 // behind long prefixes gain (2,048 tokens behind 30,720: 741 -> 682 us at head size 64, behind 63,488: 1,495 ->
 // 1,355, behind 14,336: 376 -> 363); short prompts lose, because twice as few waves, each with a chain twice as
 // long, fill the GPU worse.  The host asks for two pieces from 16,384 keys on.
+// (the registers that the bias takes would cost heads of up to 64 columns the fourth wave of a SIMD, and with it the
+// second workgroup of a CU; asked to, the compiler finds them)
 template <int TASKS, int KSPLIT, int RT = 1>
-__global__ void __launch_bounds__(64 * TASKS * KSPLIT)
+__global__ void __launch_bounds__(64 * TASKS * KSPLIT, (BIASED && HD == 64 && VD == 64 && KSPLIT > 1 && RT == 1) ? 4 : 1)
 attention_mfma_kernel(const Task* __restrict__ tasks, int n_tasks, int nkv, const uint16_t* __restrict__ q,
                       int q_stride, int nh, const int32_t* __restrict__ block_tables, int max_blocks, int window,
                       const uint16_t* __restrict__ kcache, const uint16_t* __restrict__ vcache,
@@ -264,10 +266,13 @@ attention_mfma_kernel(const Task* __restrict__ tasks, int n_tasks, int nkv, cons
     gap = (keep > 0 && window > 0 && lo > keep_end) ? lo - keep_end : 0;
   }
   auto key_of = [&](int kb) { return BIASED && kb >= keep_end ? kb + gap : kb; };
-  // the rows' slopes, in the units of the exponentials
-  float sl2[RT];
+  // The bias of a row's scores in a block is that of the lane's first key plus a ramp over its 16 keys.  The first joins
+  // the exponentials' reference point and costs nothing a score; the ramp, in the units of S before the scale, is one
+  // multiply-add a score.  (A ramp kept in registers, for the accumulators to start from, costs sixteen of them and with
+  // them the second workgroup of a CU.)
+  float per_key[RT];
 #pragma unroll
-  for (int t = 0; t < RT; ++t) sl2[t] = (BIASED && slopes != nullptr) ? slopes[head[t]] * kLog2e : 0.f;
+  for (int t = 0; t < RT; ++t) per_key[t] = (BIASED && slopes != nullptr) ? slopes[head[t]] / scale : 0.f;
 
   // page numbers: lane i asks for page (kb / PAGE + i) of the task's request; lanes 0 and 1 hold the pages that the two
   // runs of 16 keys of the block at kb may lie in (with pages of 32, 64, ... tokens both in lane 0's).  Asked for at the
@@ -418,26 +423,16 @@ attention_mfma_kernel(const Task* __restrict__ tasks, int n_tasks, int nkv, cons
       float sv[16];
       float bmax = -INFINITY;
       if constexpr (BIASED) {
-        // (a score is then in the units of the exponentials: times scale and log2 e, with its bias)
-        const float at = sl2[t] * (float)(rk + hg * 4 - p_row[t]);
 #pragma unroll
-        for (int i = 0; i < 16; ++i)
-          sv[i] = fmaf(s[t][i], sc2, fmaf(sl2[t], (float)((i >> 2) * 8 + (i & 3)), at));
-        if (edge) {
-#pragma unroll
-          for (int i = 0; i < 16; ++i) {
-            const int off = (i >> 2) * 8 + hg * 4 + (i & 3), key = rk + off;
-            const bool ok = key <= p_row[t] && (key >= lo_row[t] || key < keep) && kb + off < k_end;
-            sv[i] = ok ? sv[i] : -INFINITY;
-          }
-        }
-#pragma unroll
-        for (int i = 0; i < 16; ++i) bmax = fmaxf(bmax, sv[i]);
-      } else if (edge) {
+        for (int i = 1; i < 16; ++i) s[t][i] = fmaf(per_key[t], (float)((i >> 2) * 8 + (i & 3)), s[t][i]);
+      }
+      // the bias of this lane's first key, in the units of the exponentials
+      const float at = BIASED ? per_key[t] * sc2 * (float)(rk + hg * 4 - p_row[t]) : 0.f;
+      if (edge) {
 #pragma unroll
         for (int i = 0; i < 16; ++i) {
-          const int key = kb + (i >> 2) * 8 + hg * 4 + (i & 3);
-          const bool ok = key <= p_row[t] && key >= lo_row[t] && key < k_end;
+          const int off = (i >> 2) * 8 + hg * 4 + (i & 3), key = rk + off;
+          const bool ok = key <= p_row[t] && (key >= lo_row[t] || (BIASED && key < keep)) && kb + off < k_end;
           sv[i] = ok ? s[t][i] : -INFINITY;
           bmax = fmaxf(bmax, sv[i]);
         }
@@ -448,8 +443,12 @@ attention_mfma_kernel(const Task* __restrict__ tasks, int n_tasks, int nkv, cons
           bmax = fmaxf(bmax, sv[i]);
         }
       }
-      bmax = fmaxf(bmax, from_other_half(bmax, hg != 0));
-      if constexpr (!BIASED) bmax *= sc2;
+      if constexpr (BIASED) {
+        bmax = fmaf(bmax, sc2, at);      // (the halves' first keys differ)
+        bmax = fmaxf(bmax, from_other_half(bmax, hg != 0));
+      } else {
+        bmax = fmaxf(bmax, from_other_half(bmax, hg != 0)) * sc2;
+      }
       // The reference point m of a row's exponentials follows its maximum only in jumps: as long as no row of the
       // wave has grown by more than kSlack (in powers of two) beyond its m, m stays, the weights may exceed one (by
       // at most 2^kSlack, nothing to float32 sums or to bfloat16 weights, whose precision is relative) and the
@@ -466,10 +465,11 @@ attention_mfma_kernel(const Task* __restrict__ tasks, int n_tasks, int nkv, cons
         m[t] = m_new;
       }
       const float m_use = (m[t] == -INFINITY) ? 0.f : m[t];
+      const float less = BIASED ? at - m_use : -m_use;
       float psum = 0.f;
 #pragma unroll
       for (int i = 0; i < 16; ++i) {
-        sv[i] = __builtin_amdgcn_exp2f(BIASED ? sv[i] - m_use : fmaf(sv[i], sc2, -m_use));
+        sv[i] = __builtin_amdgcn_exp2f(fmaf(sv[i], sc2, less));
         psum += sv[i];
       }
       l[t] += psum;      // this lane's half of the row's sum; the halves meet after the last block
@@ -756,6 +756,7 @@ extern "C" int atoma_attention_mfma(const void* q, int q_stride, const void* kca
                                     const float* sinks, int keep, const float* slopes, hipStream_t stream) {
   if (n_tasks <= 0) return 0;
   if (keep < 0 || (keep > 0 && window <= 0) || (!BIASED && (keep > 0 || slopes != nullptr))) return ATOMA_ERR_SHAPE;
+  if (BIASED && !(scale > 0.f)) return ATOMA_ERR_SHAPE;      // (the bias is divided by it)
   // row_tiles: 1, or 2: the tasks that write the output cover 64 rows (Task::tiles says so), two waves a task
   if (row_tiles != 1 && !(row_tiles == 2 && kTwoPieces && ksplit == 2)) return ATOMA_ERR_SHAPE;
   if (nkv <= 0 || nh % nkv || nkv > 65535 || max_blocks <= 0 || (q_stride & 7) || (out_stride & 3) ||

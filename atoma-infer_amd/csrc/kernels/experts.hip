@@ -25,6 +25,60 @@ using namespace atoma;
 
 constexpr int kTileM = 64, kTileN = 64, kStepK = 16;
 
+// Up to 64 experts: lane e holds expert e and counts the experts that go before it (a larger score, or the same and a
+// lower index), which is its place; the scores of the others come through scalar registers, one after the other, and no
+// step waits for the one before.
+__global__ void __launch_bounds__(256)
+route_rank_kernel(const float* __restrict__ logits, int ld, int experts, int top, int32_t* __restrict__ ids,
+                  float* __restrict__ weights, int n_tokens, int score, const float* __restrict__ correction,
+                  float scale, const float* __restrict__ bias, int groups, int groups_keep) {
+  const int e = threadIdx.x & 63;
+  const int t = __builtin_amdgcn_readfirstlane(blockIdx.x * 4 + (threadIdx.x >> 6));
+  if (t >= n_tokens) return;
+  const bool real = e < experts;
+  float wt = real ? logits[(size_t)t * ld + e] + (bias != nullptr ? bias[e] : 0.f) : -INFINITY;
+  if (score == 1) {
+    const float mx = wave_max(wt);
+    wt = real ? expf(wt - mx) : 0.f;
+    wt /= wave_sum(wt);
+  } else if (score == 0) {
+    wt = 1.0f / (1.0f + expf(-wt));
+  }
+  float sc = real ? (correction != nullptr ? wt + correction[e] : wt) : -INFINITY;
+  if (!(sc == sc)) sc = -INFINITY;        // (scores that are no numbers come last: places stay a permutation)
+  auto of = [](float v, int lane) { return __uint_as_float(__builtin_amdgcn_readlane(__float_as_uint(v), lane)); };
+  if (groups > 0) {
+    const int size = experts / groups, mine = e / size;
+    float best = -INFINITY;               // of this expert's group
+    for (int g = 0; g < groups; ++g)
+      for (int i = 0; i < size; ++i) {
+        const float v = of(sc, g * size + i);
+        best = fmaxf(best, mine == g ? v : -INFINITY);
+      }
+    int before = 0;
+    for (int g = 0; g < groups; ++g) {
+      const float v = of(best, g * size);
+      before += v > best || (v == best && g < mine);
+    }
+    if (before >= groups_keep) sc = -INFINITY;
+  }
+  int place = 0;
+  for (int i = 0; i < experts; ++i) {
+    const float v = of(sc, i);
+    place += v > sc || (v == sc && i < e);
+  }
+  const bool chosen = real && place < top;
+  if (score == 2) {
+    const float mx = wave_max(chosen ? wt : -INFINITY);
+    wt = chosen ? expf(wt - mx) : 0.f;
+    wt /= wave_sum(wt);
+  }
+  if (chosen) {
+    ids[(size_t)t * top + place] = e;
+    weights[(size_t)t * top + place] = wt * scale;
+  }
+}
+
 template <bool GROUPED>
 __global__ void __launch_bounds__(256)
 route_topk_kernel(const float* __restrict__ logits, int ld, int experts, int top, int32_t* __restrict__ ids,
@@ -485,7 +539,11 @@ extern "C" int atoma_route_topk(const float* logits, int ld, int experts, int to
                                     groups_keep * (experts / groups) < top)))
     return ATOMA_ERR_SHAPE;
   const dim3 grid((n_tokens + 3) / 4), block(256);
-  if (groups > groups_keep)
+  if (groups <= groups_keep) groups = groups_keep = 0;      // (all groups are kept)
+  if (experts <= 64)
+    hipLaunchKernelGGL(route_rank_kernel, grid, block, 0, stream, logits, ld, experts, top, ids, weights, n_tokens, score,
+                       correction, scale, bias, groups, groups_keep);
+  else if (groups > 0)
     hipLaunchKernelGGL(route_topk_kernel<true>, grid, block, 0, stream, logits, ld, experts, top, ids, weights, n_tokens,
                        score, correction, scale, bias, groups, groups_keep);
   else

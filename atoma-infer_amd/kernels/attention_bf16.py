@@ -553,6 +553,8 @@ def try_attention(q, k_cache, v_cache, out, ctx, cache, scale, window, nh, nkv, 
     biased = bool(keep) or slopes is not None
     if not page_ok(page) or hd % 16 or not 16 <= hd <= 256 or vd % 16 or not 16 <= vd <= 256:
         return False
+    if biased and not scale >= 1e-6:
+        return False         # (the kernel divides the bias by the scale)
     if slopes is not None and not (slopes.dtype is torch.float32 and slopes.is_contiguous() and slopes.numel() == nh):
         raise ValueError("slopes must be contiguous float32, one per query head")
     if sinks is not None and not (sinks.dtype is torch.float32 and sinks.is_contiguous() and sinks.numel() == nh):

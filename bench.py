@@ -22,7 +22,9 @@ for the Rakuvik decoder (differential attention and a minGRU recurrence in turn,
 turn, the layers' results averaged over depth).  ``--compare bafilorn`` measures the Bafilorn decoder (a stream in
 four copies behind an embedding of token pairs; latent attention with a rotated key part, lightning attention, and
 chunked attention with tied values beside a gated linear recurrence in turn, each before a dense feed-forward with the
-square of relu) beside the Morulix of equal sizes, the closest of the other designs, and the Llama.
+square of relu) beside the Morulix of equal sizes, the closest of the other designs, and the Llama.  ``--compare
+gerorax`` measures the Gerorax decoder (attention with normed heads, distance biases and a window that keeps first keys;
+dense and grouped-routed feed-forwards in turn) beside the Somesun, the Duduvik and the Llama of equal sizes.
 
 ``--workload`` runs one of the other two workloads instead and prints ONE line of its own:
 ``serve3b``: Llama-3.2-3B sizes, 64 requests with prompt lengths uniform in [128, 4096] (seeded), 256 generated tokens
@@ -405,6 +407,39 @@ def step_bytes_duduvik(model, cfg: dict, batch: int, ctx: float) -> float:
     return total
 
 
+def gerorax_like(llama: dict, layers: int) -> dict:
+    """The Gerorax configuration beside ``llama``, ``somesun_like(llama)`` and ``duduvik_like(llama)``: the same width,
+    vocabulary and attention heads, behind a window of 1,024 keys (the Somesun's chunks) and the first 4; feed-forwards in
+    turn dense of the Llama's width and routed experts of the Somesun's sizes in eight groups (half of them kept) with a
+    shared one; all layers one pass of a loop."""
+    w, nh, nkv = llama["hidden_size"], llama["num_attention_heads"], llama["num_key_value_heads"]
+    hd = w // nh
+    ff = 2048 if w <= 2048 else 4096
+    top = llama["intermediate_size"] // ff
+    moe = {"kind": "moe", "expert": {"ff": ff, "limit": 7.0}, "shared": {"ff": ff, "limit": 7.0},
+           "router": {"experts": 8 * top, "top": top, "groups": {"count": 8, "keep": 4}}}
+    att = {"dim": hd, "heads": nh, "kv_heads": nkv, "vdim": hd, "scale": hd ** -0.5, "mask": {"keep_first": 4, "size": 1024}}
+    dense = {"kind": "dense", "ff": llama["intermediate_size"]}
+    return {"architecture": "Gerorax", "embedding": {"scale": 1.0}, "residual_mult": 0.5,
+            "layers": [{"type": "attention", "mixer": att, "mlp": moe if i % 2 else dense} for i in range(layers)],
+            "loop": {"start": 0, "stop": layers, "times": 1}, "norm": {"eps": 1e-5}, "vocab": llama["vocab_size"], "width": w,
+            "max_positions": llama["max_position_embeddings"]}
+
+
+def step_bytes_gerorax(model, cfg: dict, batch: int, ctx: float) -> float:
+    """Bytes a decode step of ``batch`` requests at context ``ctx`` has to read: every dense matrix once, the experts
+    that ``batch`` tokens are expected to choose between them, the keys and values of the window and the kept ones."""
+    total = float(model.weight_bytes())
+    for l in cfg["layers"]:
+        m, f = l["mixer"], l["mlp"]
+        seen = min(ctx, m["mask"]["size"] + m["mask"]["keep_first"]) if m.get("mask") else ctx
+        total += batch * seen * 2.0 * m["kv_heads"] * (m["dim"] + m["vdim"])
+        if f and f["kind"] == "moe":
+            e, top = f["router"]["experts"], f["router"]["top"]
+            total += (e * (1.0 - (1.0 - top / e) ** batch) - top) * 2.0 * 3 * cfg["width"] * f["expert"]["ff"]
+    return total
+
+
 def compare_main(args) -> int:
     import torch
     import atoma_infer_amd  # noqa: F401
@@ -415,13 +450,15 @@ def compare_main(args) -> int:
     llama = dict(dict(LLAMA_1B, **OTHER_SIZES.get(sizes, {})), num_hidden_layers=layers)
     design = args.compare
     sun = {"somesun": somesun_like, "morulix": morulix_like, "rakuvik": rakuvik_like,
-           "bafilorn": bafilorn_like, "duduvik": duduvik_like}[design](llama, layers)
+           "bafilorn": bafilorn_like, "duduvik": duduvik_like, "gerorax": gerorax_like}[design](llama, layers)
     out = {}
     pairs = [("llama", llama), (design, sun)]
     if design == "bafilorn":      # also the closest of the other designs, at the same sizes
         pairs.insert(1, ("morulix", morulix_like(llama, layers)))
     if design == "duduvik":
         pairs[1:1] = [("somesun", somesun_like(llama, layers)), ("bafilorn", bafilorn_like(llama, layers))]
+    if design == "gerorax":
+        pairs[1:1] = [("somesun", somesun_like(llama, layers)), ("duduvik", duduvik_like(llama, layers))]
     for name, cfg in pairs:
         if args.only and args.only != name:
             continue
@@ -440,6 +477,8 @@ def compare_main(args) -> int:
                 nbytes = step_bytes_bafilorn(model, cfg, b, ctx)
             elif name == "duduvik":
                 nbytes = step_bytes_duduvik(model, cfg, b, ctx)
+            elif name == "gerorax":
+                nbytes = step_bytes_gerorax(model, cfg, b, ctx)
             elif name == "morulix":
                 nbytes = step_bytes_morulix(model, cfg, b, ctx)
             elif name == "rakuvik":
@@ -526,9 +565,9 @@ def main() -> int:
     ap.add_argument("--top-p", type=float, default=1.0)
     ap.add_argument("--workload", choices=["decode", *WORKLOADS], default="decode",
                     help="decode: the default run; serve3b, long8b: the other two workloads, one line of their own")
-    ap.add_argument("--compare", choices=["somesun", "morulix", "rakuvik", "bafilorn", "duduvik"], default=None,
+    ap.add_argument("--compare", choices=["somesun", "morulix", "rakuvik", "bafilorn", "duduvik", "gerorax"], default=None,
                     help="measure that design at --sizes (1b, 3b) beside the Llama of equal sizes, one line of its own")
-    ap.add_argument("--only", choices=["llama", "somesun", "morulix", "rakuvik", "bafilorn", "duduvik"], default=None,
+    ap.add_argument("--only", choices=["llama", "somesun", "morulix", "rakuvik", "bafilorn", "duduvik", "gerorax"], default=None,
                     help="with --compare: one of its models")
     ap.add_argument("--requests", type=int, default=0, help="requests of a --workload run (default: the workload's)")
     ap.add_argument("--no-peaks", action="store_true", help="skip the probes of what the GPU delivers")
