@@ -82,10 +82,11 @@ STANDARD_HEAD_SIZES = tuple(range(16, 257, 16))
 # (head size, tokens a page) beyond pages of 16 tokens that the build check compiles too: the head sizes of the Llamas
 # with pages of 32 and 64 tokens, and what the tests run; any other pair is compiled when a cache first has it
 LARGER_PAGE_MODULES = tuple((hd, page) for hd in (32, 48, 64, 128) for page in (32, 64)) + ((64, 48), (80, 48))
-# (head size, value size) of attention with scores biased by distance, or windows that keep a request's first keys,
-# that the build check compiles: those that the tests and the bench run
-BIASED_MODULES = ((16, 16), (16, 48), (32, 32), (48, 16), (48, 80), (64, 64), (64, 128), (96, 96), (128, 64), (128, 128),
-                  (160, 32), (192, 192), (208, 64), (64, 208), (256, 256))
+# (head size, value size, tokens a page) of attention with scores biased by distance, or windows that keep a request's
+# first keys, that the build check compiles: those that the tests and the bench run
+BIASED_MODULES = tuple((hd, vd, 16) for hd in (16, 32, 64) for vd in (16, 32, 64)) + (
+    (32, 48, 16), (48, 32, 16), (48, 80, 16), (64, 128, 16), (96, 96, 16), (128, 64, 16), (128, 128, 16), (160, 32, 16),
+    (192, 192, 16), (208, 64, 16), (64, 208, 16), (256, 256, 16), (64, 64, 32), (64, 64, 64), (32, 48, 48), (128, 64, 32))
 
 
 def _lock_for(name: str) -> threading.Lock:
@@ -246,8 +247,8 @@ def build_all(head_sizes: Sequence[int] = STANDARD_HEAD_SIZES) -> List[str]:
              for hd in head_sizes]
     jobs += [(attention_bf16.module_name(hd, page), ("attention_mfma.hip",), attention_bf16.module_defines(hd, page))
              for hd, page in LARGER_PAGE_MODULES]
-    jobs += [(attention_bf16.module_name(hd, vd=vd, biased=True), ("attention_mfma.hip",),
-              attention_bf16.module_defines(hd, vd=vd, biased=True)) for hd, vd in BIASED_MODULES]
+    jobs += [(attention_bf16.module_name(hd, page, vd, True), ("attention_mfma.hip",),
+              attention_bf16.module_defines(hd, page, vd, True)) for hd, vd, page in BIASED_MODULES]
     jobs += [linear_attention_module(dp) for dp in LINEAR_ATTENTION_SIZES]
     with ThreadPoolExecutor(min(8, len(jobs))) as pool:
         futs = [pool.submit(load_hip_module, n, src, d, force_build=True) for n, src, d in jobs]

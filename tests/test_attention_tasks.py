@@ -6,7 +6,7 @@ import pytest
 from atoma_infer_amd.kernels import attention_bf16 as A
 
 
-def coverage(arr, meta, starts, counts, group, window):
+def coverage(arr, meta, starts, counts, group, window, keep=0):
     n_main, n_comb, n_part, waves, tiles, merge = meta
     assert waves in (1, 2, 4, 8) and tiles in (1, 2) and (tiles == 1 or waves == 2)
     main, comb = arr[:n_main], arr[n_main:]
@@ -19,17 +19,24 @@ def coverage(arr, meta, starts, counts, group, window):
             continue
         assert tok_base == int(np.sum(counts[:e])) and count == counts[e] and pos0 == starts[e]
         assert kb % 32 == 0 and kb < ke
+        # with kept keys a task counts along its tile's walk: the blocks below the kept ones' end, then on from the window of
+        # the tile's first token
+        lo32 = max(0, pos0 + tok0 - window + 1) // 32 * 32 if window else 0
+        keep_end = -(-keep // 32) * 32
+        gap = max(0, lo32 - keep_end) if keep else 0
         # a task that writes the output covers `tiles` pieces of 32 rows, one that leaves a partial result one
         assert (max(pieces, 1) == tiles) if dest < 0 else pieces <= 1
         n_rows = 32 * max(pieces, 1)
         rows = [(tok0 + r % qt, r // qt) for r in range(row0, row0 + n_rows) if r // qt < group and tok0 + r % qt < count]
         assert rows
+        real = [(kb, ke)] if not gap or ke <= keep_end else [(kb + gap, ke + gap)] if kb >= keep_end else \
+            [(kb, keep_end), (keep_end + gap, ke + gap)]
         if dest < 0:
             for row in rows:
-                seen.setdefault((e,) + row, []).append((kb, ke))
+                seen.setdefault((e,) + row, []).extend(real)
         else:
             assert 0 <= dest < n_part and dest not in parts
-            parts[dest] = (e, rows, (kb, ke))
+            parts[dest] = (e, rows, real)
     for t in comb:
         e, tok0, qt, row0, _, _, dest, n_parts, *_ = (int(x) for x in t)
         rows = [(tok0 + r % qt, r // qt) for r in range(row0, row0 + 32) if r // qt < group and tok0 + r % qt < counts[e]]
@@ -37,7 +44,7 @@ def coverage(arr, meta, starts, counts, group, window):
             pe, prows, rng = parts.pop(p)
             assert pe == e and prows == rows
             for row in rows:
-                seen.setdefault((e,) + row, []).append(rng)
+                seen.setdefault((e,) + row, []).extend(rng)
     assert not parts, "a partial result that nobody merges"
     for e in range(len(starts)):
         for tok in range(counts[e]):
@@ -46,9 +53,20 @@ def coverage(arr, meta, starts, counts, group, window):
             for h in range(group):
                 ranges = sorted(seen[(e, tok, h)])
                 # ranges tile a span that holds every visible key, without overlap
-                assert ranges[0][0] <= lo and ranges[-1][1] >= p + 1
+                if not keep:
+                    assert ranges[0][0] <= lo and ranges[-1][1] >= p + 1
+                    for (a, b), (c, d) in zip(ranges, ranges[1:]):
+                        assert b == c
+                    continue
+                # ... or, with kept keys, the two spans that hold them and the window, nothing twice
                 for (a, b), (c, d) in zip(ranges, ranges[1:]):
-                    assert b == c
+                    assert b <= c
+                walked = np.zeros(p + 200, dtype=bool)
+                for a, b in ranges:
+                    walked[a:b] = True
+                assert walked[lo: p + 1].all() and walked[: min(keep, p + 1)].all()
+                # and not much else: whole blocks at both ends of the gap, and the windows of a tile's other tokens
+                assert walked[: p + 1].sum() <= min(p + 1, window + keep + 62 + 128)
 
 
 @pytest.mark.parametrize("seed", range(30))
@@ -90,6 +108,38 @@ def test_decode_builder_equals_the_general_one(seed):
     # sizes depend on (entries, bucket) alone
     other = rng.integers(0, bucket, size=s).astype(np.int32)
     assert A.build_tasks(other, counts, group, window, bucket, kv_heads=8)[1] == mf
+
+
+@pytest.mark.parametrize("seed", range(40))
+def test_tasks_of_windows_that_keep_first_keys_cover_them_and_the_window_once(seed, monkeypatch):
+    rng = np.random.default_rng(900 + seed)
+    s = int(rng.integers(1, 9))
+    group = int(rng.choice([1, 3, 4, 8, 40]))
+    window, keep = int(rng.choice([1, 2, 32, 50, 700])), int(rng.choice([1, 4, 31, 32, 33, 200]))
+    counts = rng.choice([1, 1, 2, 7, 33, 150], size=s).astype(np.int32)
+    starts = rng.choice([0, 3, 31, 32, 33, 64, 97, 700, 1501, 2400], size=s).astype(np.int32)
+    args = dict(kv_heads=8, keep=keep)
+    arr, meta = A.build_tasks(starts, counts, group, window, **args)
+    coverage(arr, meta, starts, counts, group, window, keep)
+    monkeypatch.setattr(A, "TWO_PIECES_MIN_KEYS", int(rng.choice([0, 1500])))
+    fast, mf = A.build_tasks(starts, counts, group, window, max_waves=8, row_tiles=2, **args)
+    coverage(fast, mf, starts, counts, group, window, keep)
+    slow, ms = A.build_tasks(starts, counts, group, window, vectorized=False, max_waves=8, row_tiles=2, **args)
+    assert mf == ms and sorted(map(tuple, fast.tolist())) == sorted(map(tuple, slow.tolist()))
+    # decoded tokens: both builders, chunks and whole ranges, the same counts for any starts below the bucket
+    one = np.ones(s, dtype=np.int32)
+    bucket = -(-int(starts.max() + 1) // 256) * 256
+    for waves in (2, 8):
+        fast, mf = A.build_tasks(starts, one, group, window, bucket, max_waves=waves, **args)
+        coverage(fast, mf, starts, one, group, window, keep)
+        other = rng.integers(0, bucket, size=s).astype(np.int32)
+        again, ma = A.build_tasks(other, one, group, window, bucket, max_waves=waves, **args)
+        coverage(again, ma, other, one, group, window, keep)
+        assert ma == mf
+    fast, mf = A.build_tasks(starts, one, group, window, bucket, **args)
+    slow, ms = A.build_tasks(starts, one, group, window, bucket, vectorized=False, **args)
+    live = fast[:, 0] >= 0
+    assert mf == ms and np.array_equal(live, slow[:, 0] >= 0) and np.array_equal(fast[live], slow[live])
 
 
 @pytest.mark.parametrize("seed", range(8))

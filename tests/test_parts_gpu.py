@@ -158,8 +158,8 @@ def test_attention_part(act, nh, nkv, hd, width, window):
 @pytest.mark.parametrize("window", [None, 24])
 def test_an_encoding_that_biases_scores_by_distance(act, window):
     """A position encoding defined here that rotates nothing and gives each head a slope: the score of the key at j
-    for the query at p gains slope * (j - p).  The framework's attention takes it through its general kernel; the
-    plain formula is written out below (softmax over the visible keys of q.k * scale + slope * (j - p))."""
+    for the query at p gains slope * (j - p).  The framework's attention takes it (in bfloat16 through the matrix-core
+    kernel); the plain formula is written out below (softmax over the visible keys of q.k * scale + slope * (j - p))."""
     from atoma_infer_amd.cache.pool import LayerCache
     from atoma_infer_amd.parts import PagedAttention, PositionEncoding
 
@@ -180,7 +180,7 @@ def test_an_encoding_that_biases_scores_by_distance(act, window):
            ("v_proj.weight", (nkv * hd, width)), ("o_proj.weight", (width, nh * hd)))}
     part = PagedAttention(width, nh, nkv, hd, Slopes(), window)
     part.load(getter(ws), torch.device(DEV), act)
-    assert part.step_planner(page, act) is None              # the general kernel needs no plan
+    assert (part.step_planner(page, act) is None) == (act is torch.float32)      # the general kernel needs no plan
     x = torch.randn(n, width, generator=g).to(act)
     xf, w = x.double(), {k: v.double() for k, v in ws.items()}
     q = (xf @ w["q_proj.weight"].T).view(n, nh, hd)
