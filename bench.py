@@ -411,7 +411,8 @@ def gerorax_like(llama: dict, layers: int) -> dict:
     """The Gerorax configuration beside ``llama``, ``somesun_like(llama)`` and ``duduvik_like(llama)``: the same width,
     vocabulary and attention heads, behind a window of 1,024 keys (the Somesun's chunks) and the first 4; feed-forwards in
     turn dense of the Llama's width and routed experts of the Somesun's sizes in eight groups (half of them kept) with a
-    shared one; all layers one pass of a loop."""
+    shared one; all layers one pass of a loop.  The embedding's factor makes its random rows as large as the sinusoid:
+    with small ones the positions alone would decide, and requests side by side would choose the same experts."""
     w, nh, nkv = llama["hidden_size"], llama["num_attention_heads"], llama["num_key_value_heads"]
     hd = w // nh
     ff = 2048 if w <= 2048 else 4096
@@ -420,7 +421,7 @@ def gerorax_like(llama: dict, layers: int) -> dict:
            "router": {"experts": 8 * top, "top": top, "groups": {"count": 8, "keep": 4}}}
     att = {"dim": hd, "heads": nh, "kv_heads": nkv, "vdim": hd, "scale": hd ** -0.5, "mask": {"keep_first": 4, "size": 1024}}
     dense = {"kind": "dense", "ff": llama["intermediate_size"]}
-    return {"architecture": "Gerorax", "embedding": {"scale": 1.0}, "residual_mult": 0.5,
+    return {"architecture": "Gerorax", "embedding": {"scale": 50.0}, "residual_mult": 0.5,
             "layers": [{"type": "attention", "mixer": att, "mlp": moe if i % 2 else dense} for i in range(layers)],
             "loop": {"start": 0, "stop": layers, "times": 1}, "norm": {"eps": 1e-5}, "vocab": llama["vocab_size"], "width": w,
             "max_positions": llama["max_position_embeddings"]}
